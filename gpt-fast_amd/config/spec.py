@@ -145,6 +145,30 @@ class GatedDeltaSpec:
 
 
 @dataclass(frozen=True)
+class StateSpaceSpec:
+    """Recurrent mixer with a matrix state per head and a decay that depends on the token
+    (state-space duality, the cell of Mamba-2).  One projection gives a gate z and x
+    (``n_heads * value_dim`` each), B and C (``n_groups`` of ``state`` each) and one step size per
+    head; head h uses group ``h // (n_heads / n_groups)`` of B and C.  Each channel of x, B and C
+    passes a causal convolution over ``conv_taps`` tokens (with a bias, zeros before the start)
+    and silu; ``dt = softplus(. + dt_bias)``; per head a float32 state ``S [state, value_dim]``,
+    zero at a sequence's start: ``S <- exp(-exp(A_log) dt) S + dt B x^T; y = S^T C + D x``.  The
+    heads' results side by side are multiplied by silu(z) FIRST and then divided, in
+    ``norm_groups`` equal parts, each by its own root mean square (``eps``), times a weight per
+    element, and projected out.  The convolution's last ``conv_taps - 1`` inputs are part of the
+    sequence's state."""
+    dim: int
+    n_heads: int
+    value_dim: int
+    state: int
+    n_groups: int
+    conv_taps: int
+    norm_groups: int
+    eps: float
+    kind: str = "state_space"
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Several mixers side by side that read the same input: ``branches`` = ((name, spec), ...),
     each any mixer spec.  The result is the mean of the branches' results, each first divided
@@ -218,10 +242,12 @@ class LatentAttentionSpec:
     latent of ``kv_rank`` (RMS-normed) and one rotated key part of ``rot_dim`` that all heads
     share; a head's plain key is ``w_uk`` of the latent, its value ``w_uv`` of it
     (``value_dim``).  score = (q_plain . k_plain + q_rot . k_rot) * scale.  ``position``
-    rotates the first ``position.rotary_dim`` elements of the rotated parts.  ``window`` W:
-    keys at distance < W only.  The cache holds the latent and the rotated key part.
+    rotates the first ``position.rotary_dim`` elements of the rotated parts (any layout and
+    scaling of ``PositionSpec``).  ``window`` W: keys at distance < W only.  The cache holds the
+    latent and the rotated key part.
     ``q_rank`` None: the query has no latent, one projection takes x straight to the heads.
-    ``rot_dim`` 0: no rotated part."""
+    ``rot_dim`` 0: no rotated part.  ``head_gate``: head h's result is multiplied by
+    ``sigmoid(w_g x)_h`` (one number per token and head)."""
     dim: int
     n_heads: int
     head_dim: int
@@ -233,6 +259,7 @@ class LatentAttentionSpec:
     eps: float
     position: PositionSpec
     window: Optional[int] = None
+    head_gate: bool = False
     kind: str = "latent_attention"
 
 
@@ -382,7 +409,11 @@ class LayerSpec:
     the norm stands after the sum, ``x <- out_norm(residual_scale * x + ls * sublayer(read(x)))``:
     ``mixer_norm`` / ``feed_forward_norm`` say how a sublayer reads the stream (kind "none": the
     stream itself), ``mixer_out_norm`` / ``feed_forward_out_norm`` are the norms of the sums, and
-    ``layer_scale`` gives each sublayer's result a stored weight per element ``ls``."""
+    ``layer_scale`` gives each sublayer's result a stored weight per element ``ls``.
+    In the "hyper_connected" arrangement ``streams`` copies x_1 .. x_S stand in place of one
+    stream (hyper-connections): a sublayer reads ``norm(sum_s in[s] x_s)`` and gives y, and all
+    streams move at once, ``x_t <- sum_s mix[s, t] x_s + out[t] y``, with stored numbers ``in [S]``,
+    ``out [S]`` and ``mix [S, S]`` (from, to) per sublayer."""
     name: str
     mixer: object
     mixer_norm: NormSpec
@@ -403,6 +434,11 @@ class LayerSpec:
     result_gate: bool = False
     mixer_gate_name: str = "mixer_gate"
     feed_forward_gate_name: str = "feed_forward_gate"
+    # "hyper_connected": the number of streams that stand in place of one, and the names of the
+    # weights with which each sublayer reads and writes them
+    streams: Optional[int] = None
+    mixer_streams_name: str = "mixer_streams"
+    feed_forward_streams_name: str = "feed_forward_streams"
     # "post_norm": the stream's factor in the sum, and a weight per element on each result
     residual_scale: float = 1.0
     layer_scale: bool = False
@@ -446,13 +482,23 @@ class ModelPlan:
     # further parts that add to the embedded rows (``PairEmbeddingSpec``); each may keep state
     # per sequence in a cache entry of its own
     input_adds: Tuple[object, ...] = ()
+    # the residual stream is this many copies of the embedded rows, which "hyper_connected"
+    # layers read and write; their sum is what the final norm reads.  None: one stream, the plain
+    # residual sum
+    streams: Optional[int] = None
     logit_scale: Optional[float] = None         # logits are multiplied by this,
     logit_softcap: Optional[float] = None       # then capped: cap * tanh(logits / cap)
 
     def validate(self) -> None:
         if not self.layers:
             raise ValueError("a model plan needs at least one layer")
+        for i, layer in enumerate(self.layers):
+            mine = getattr(layer, "streams", None)
+            if mine != self.streams:
+                raise ValueError(f"layer {i} works on {mine} streams, the plan has {self.streams}")
         for n, run in enumerate(self.order):
+            if self.streams is not None and getattr(run, "enter", None) is not None:
+                raise ValueError(f"order[{n}].enter: a step on the stream has no meaning for several")
             if not 0 <= run.layer < len(self.layers):
                 raise ValueError(f"order[{n}] names layer {run.layer}, "
                                  f"but there are {len(self.layers)} layers")

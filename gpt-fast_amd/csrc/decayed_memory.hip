@@ -412,3 +412,108 @@ extern "C" int gfa_row_norm_gate(const float* o, const float* weight, int weight
             o, weight, weight_width, proj, row_width, g_off, (float*)y, width, groups, gate_act, eps);
     return GFA_LAUNCH_RESULT();
 }
+
+// --------------------------------------------------------------------------------------
+// The same with the gate BEFORE the norm (the output of a state-space cell):
+//     u = o[t, :] * gate(g[t, :]);   y[t, :] = u * rsqrt(mean_over_part(u^2) + eps) * weight[:]
+// One workgroup per (part of a row, token); a thread keeps up to NV * 4 elements in registers
+// (VEC: the parts' places and sizes are multiples of four), and works the rest out twice.
+template <typename T, bool VEC, int NV>
+__global__ __launch_bounds__(256) void gate_row_norm_kernel(
+        const float* __restrict__ o, const float* __restrict__ weight, int weight_width,
+        const float* __restrict__ proj, int row_width, int g_off, T* __restrict__ y, int width,
+        int groups, int gate_act, float eps) {
+    __shared__ float scratch[16];
+    const size_t t = blockIdx.y;
+    const int part = width / groups, base = blockIdx.x * part;
+    const float* src = o + t * width + base;
+    const float* gate = proj + t * row_width + g_off + base;
+    T* dst = y + t * width + base;
+    auto gated = [&](float v, float g) {
+        const float sg = 1.f / (1.f + expf(-g));
+        return v * (gate_act ? g * sg : sg);
+    };
+    float ss = 0.f;
+    if (VEC) {
+        const int n4 = part >> 2;
+        float4 u[NV];
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int e = threadIdx.x + i * 256;
+            u[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (e < n4) {
+                const float4 v = *(const float4*)(src + 4 * e), g = *(const float4*)(gate + 4 * e);
+                u[i] = make_float4(gated(v.x, g.x), gated(v.y, g.y), gated(v.z, g.z), gated(v.w, g.w));
+            }
+            ss = fmaf(u[i].x, u[i].x, ss);
+            ss = fmaf(u[i].y, u[i].y, ss);
+            ss = fmaf(u[i].z, u[i].z, ss);
+            ss = fmaf(u[i].w, u[i].w, ss);
+        }
+        const float r = rsqrtf(block_sum(ss, scratch) / (float)part + eps);
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int e = threadIdx.x + i * 256;
+            if (e < n4) {
+                const float4 w = weight ? *(const float4*)(weight + (base + 4 * e) % weight_width)
+                                        : make_float4(1.f, 1.f, 1.f, 1.f);
+                store_from_float(dst + 4 * e + 0, u[i].x * r * w.x);
+                store_from_float(dst + 4 * e + 1, u[i].y * r * w.y);
+                store_from_float(dst + 4 * e + 2, u[i].z * r * w.z);
+                store_from_float(dst + 4 * e + 3, u[i].w * r * w.w);
+            }
+        }
+        return;
+    }
+    for (int d = threadIdx.x; d < part; d += 256) {
+        const float u = gated(src[d], gate[d]);
+        ss = fmaf(u, u, ss);
+    }
+    const float r = rsqrtf(block_sum(ss, scratch) / (float)part + eps);
+    for (int d = threadIdx.x; d < part; d += 256)
+        store_from_float(dst + d, gated(src[d], gate[d]) * r * (weight ? weight[(base + d) % weight_width] : 1.f));
+}
+
+template <typename T>
+static int launch_gate_row_norm(const float* o, const float* weight, int weight_width, const float* proj,
+                                int row_width, int g_off, T* y, int n_tokens, int width, int groups,
+                                int gate_act, float eps, hipStream_t stream) {
+    const int part = width / groups;
+    const dim3 grid(groups, n_tokens);
+    const bool vec = part % 4 == 0 && row_width % 4 == 0 && g_off % 4 == 0 && part <= 16384
+        && (!weight || weight_width % 4 == 0) && (size_t)o % 16 == 0 && (size_t)proj % 16 == 0
+        && (size_t)weight % 16 == 0;
+#define GRN_GO(VEC, NV) gate_row_norm_kernel<T, VEC, NV><<<grid, 256, 0, stream>>>( \
+        o, weight, weight_width, proj, row_width, g_off, y, width, groups, gate_act, eps)
+    if (!vec) GRN_GO(false, 1);
+    else if (part <= 1024) GRN_GO(true, 1);
+    else if (part <= 2048) GRN_GO(true, 2);
+    else if (part <= 4096) GRN_GO(true, 4);
+    else if (part <= 8192) GRN_GO(true, 8);
+    else GRN_GO(true, 16);
+#undef GRN_GO
+    return GFA_LAUNCH_RESULT();
+}
+
+extern "C" int gfa_gate_row_norm(const float* o, const float* weight, int weight_width,
+                                 const float* proj, int row_width, int g_off, void* y, int y_bf16,
+                                 int n_tokens, int width, int groups, int gate_act, float eps,
+                                 hipStream_t stream) {
+    if (n_tokens <= 0) return 0;
+    if (groups < 1 || width % groups || n_tokens > 65535 * 64
+            || (weight && (weight_width < 1 || width % weight_width)))
+        return (int)hipErrorInvalidValue;
+    // a launch's second dimension ends at 65,535
+    for (int t0 = 0; t0 < n_tokens; t0 += 65535) {
+        const int n = n_tokens - t0 < 65535 ? n_tokens - t0 : 65535;
+        const float* op = o + (size_t)t0 * width;
+        const float* pp = proj + (size_t)t0 * row_width;
+        const int rc = y_bf16
+            ? launch_gate_row_norm<bf16_t>(op, weight, weight_width, pp, row_width, g_off,
+                                           (bf16_t*)y + (size_t)t0 * width, n, width, groups, gate_act, eps, stream)
+            : launch_gate_row_norm<float>(op, weight, weight_width, pp, row_width, g_off,
+                                          (float*)y + (size_t)t0 * width, n, width, groups, gate_act, eps, stream);
+        if (rc) return rc;
+    }
+    return 0;
+}

@@ -11,77 +11,14 @@
 //
 // Head h of v, beta, g and o uses head h / (H / G) of q and k.  Everything here is float
 // arithmetic.  One slot's state: S [H][dk][dv], then the convolutions' tails [K - 1][C], oldest
-// first, C = 2 G dk + H dv channels in the order q, k, v.
+// first, C = 2 G dk + H dv channels in the order q, k, v.  The convolutions are short_conv.hip's.
 #include "common.h"
 
 #define GD_THREADS 256
 #define GD_COLS 32                      // columns of S (elements of v) per workgroup
 #define GD_GROUPS (GD_THREADS / GD_COLS)
-#define GD_MAX_TAPS 16
 
-__device__ __forceinline__ float gd_silu(float z) { return z / (1.f + expf(-z)); }
 __device__ __forceinline__ float gd_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
-// y[n, c] = silu(sum_j taps[c, j] x[n - (K - 1) + j, c]) over the tokens of n's own sequence;
-// inputs before the step come from the sequence's tail, which is left as it is.  The
-// convolved channels are the first C columns of a row of proj.  One thread per (token, channel).
-__global__ __launch_bounds__(256) void short_conv_kernel(
-        const float* __restrict__ proj, int row_width, const float* __restrict__ taps, int K, int C,
-        const float* __restrict__ state, size_t slot_stride, size_t tail_off,
-        const int* __restrict__ tok_seq, const int* __restrict__ q_start,
-        const int* __restrict__ slots, float* __restrict__ y, int n_tokens) {
-    const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
-    if (idx >= (long long)n_tokens * C) return;
-    const int n = (int)(idx / C), c = (int)(idx - (long long)n * C);
-    const int b = tok_seq[n];
-    const int first = q_start[b];
-    const float* tail = state + (size_t)slots[b] * slot_stride + tail_off;
-    float acc = 0.f;
-    for (int j = 0; j < K; ++j) {
-        const int src = n - (K - 1) + j;               // a row of this step, if it is the sequence's
-        const float x = src >= first ? proj[(size_t)src * row_width + c]
-                                     : tail[(size_t)(K - 1 + src - first) * C + c];
-        acc = fmaf(taps[(size_t)c * K + j], x, acc);
-    }
-    y[(size_t)n * C + c] = gd_silu(acc);
-}
-
-// The tails after the step: the last K - 1 of (old tail, the step's inputs).  One thread per
-// (sequence, channel) reads its old entries before it writes.
-__global__ __launch_bounds__(256) void conv_tail_kernel(
-        const float* __restrict__ proj, int row_width, int K, int C, float* __restrict__ state,
-        size_t slot_stride, size_t tail_off, const int* __restrict__ q_start,
-        const int* __restrict__ slots, int n_seqs) {
-    const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
-    if (idx >= (long long)n_seqs * C) return;
-    const int b = (int)(idx / C), c = (int)(idx - (long long)b * C);
-    const int first = q_start[b], L = q_start[b + 1] - first;
-    float* tail = state + (size_t)slots[b] * slot_stride + tail_off;
-    float old[GD_MAX_TAPS];
-    for (int i = 0; i < K - 1; ++i) old[i] = tail[(size_t)i * C + c];
-    for (int i = 0; i < K - 1; ++i) {
-        const int at = L + i;                           // in (old tail, inputs of the step)
-        tail[(size_t)i * C + c] = at < K - 1 ? old[at]
-                                             : proj[(size_t)(first + at - (K - 1)) * row_width + c];
-    }
-}
-
-extern "C" int gfa_short_conv(const float* proj, int row_width, const float* taps, int K, int C,
-                              float* state, size_t slot_stride, size_t tail_off, const int* tok_seq,
-                              const int* q_start, const int* slots, float* y, int n_tokens, int n_seqs,
-                              hipStream_t stream) {
-    if (n_tokens <= 0 || n_seqs <= 0) return 0;
-    if (K < 1 || K > GD_MAX_TAPS || C < 1 || C > row_width) return (int)hipErrorInvalidValue;
-    const long long units = (long long)n_tokens * C;
-    short_conv_kernel<<<(unsigned)((units + 255) / 256), 256, 0, stream>>>(
-        proj, row_width, taps, K, C, state, slot_stride, tail_off, tok_seq, q_start, slots, y, n_tokens);
-    if (K > 1) {
-        const long long tails = (long long)n_seqs * C;
-        conv_tail_kernel<<<(unsigned)((tails + 255) / 256), 256, 0, stream>>>(
-            proj, row_width, K, C, state, slot_stride, tail_off, q_start, slots, n_seqs);
-    }
-    return GFA_LAUNCH_RESULT();
-}
 
 struct GDShape {
     int H, G, dk, dv;

@@ -9,6 +9,7 @@
 //     s_h(j) = s_h(j) - r1[h] ln(1 + r2[h] (i - j))                     (r1, r2 optional)
 //     z_h(j) = sum_h' talk[h, h'] s_h'(j)                               (talk optional)
 //     out_h  = sum_j softmax_j(z_h)(j) v_g(j)
+//     out_h  = out_h sigmoid(gate[token, h])                            (gate optional)
 // With a sink the softmax's denominator has one more term, exp(0): a key of score zero that
 // carries no value (the running maximum starts at 0 and the running sum at 1).
 // row(n) = lookup[n] for n < n_lookup, else bias_rows - 1 (the host fills the lookup table).
@@ -32,6 +33,8 @@ struct SAShape {
     float scale, softcap;
     int bias_rows, n_lookup;
     int sink;
+    const float* gate;                           // a row of pre-activations per token, or null
+    long long gate_tok;                          // floats from one token's row to the next
 };
 
 template <typename T> struct Pack8;
@@ -193,10 +196,11 @@ __global__ __launch_bounds__(SA_THREADS) void scored_attention_kernel(
         const int h = h0 + wave + SA_WAVES * i;
         if (h >= s.H) continue;
         T* o = out + (size_t)n * s.o_tok + (size_t)h * s.o_head;
+        const float open = s.gate ? 1.f / (1.f + expf(-s.gate[(size_t)n * s.gate_tok + h])) : 1.f;
 #pragma unroll
         for (int e = 0; e < VPT; ++e) {
             const int d = lane + 64 * e;
-            if (d < s.vd) store_from_float(o + d, acc[i][e] / l[i]);
+            if (d < s.vd) store_from_float(o + d, acc[i][e] / l[i] * open);
         }
     }
 }
@@ -256,13 +260,13 @@ extern "C" int gfa_scored_attention(const void* q, const void* k_pages, const vo
                                     const float* r2, int sink, void* out, int n_tokens,
                                     int H, int G, int hd, int vd, long long q_tok, long long q_head,
                                     long long o_tok, long long o_head, float scale, float softcap,
-                                    int bias_rows, int n_lookup, int window, int is_bf16,
-                                    hipStream_t stream) {
+                                    int bias_rows, int n_lookup, int window, const float* gate,
+                                    long long gate_tok, int is_bf16, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (G <= 0 || H % G || hd <= 0 || vd <= 0 || vd > 512) return (int)hipErrorInvalidValue;
     if ((r1 == nullptr) != (r2 == nullptr)) return (int)hipErrorInvalidValue;
     SAShape s{H, G, hd, vd, q_tok, q_head, o_tok, o_head, table_stride, window, scale, softcap,
-              bias_rows, n_lookup, sink ? 1 : 0};
+              bias_rows, n_lookup, sink ? 1 : 0, gate, gate_tok};
     if (is_bf16)
         return sa_dispatch<bf16_t>(q, k_pages, v_pages, tok_seq, tok_pos, table, temperature, bias,
                                    lookup, talk, r1, r2, out, n_tokens, s, stream);
@@ -569,7 +573,8 @@ __global__ __launch_bounds__(MAXT) void scored_attention_mfma_kernel(
                         o[dt][j] = fmaf(theirs[32 + (dt * 16 + lg * 4 + j) * 16 + li], f, o[dt][j]);
         }
     }
-    const float inv = l > 0.f ? 1.f / l : 0.f;
+    float inv = l > 0.f ? 1.f / l : 0.f;
+    if (s.gate) inv /= 1.f + expf(-s.gate[(size_t)(q0 + tok) * s.gate_tok + head]);
     if (!row_ok) return;
     bf16_t* orow = out + (size_t)(q0 + tok) * s.o_tok + (size_t)head * s.o_head;
 #pragma unroll
@@ -661,7 +666,8 @@ extern "C" int gfa_scored_attention_mfma(const void* q, const void* k_pages, con
                                          void* out, int n_seqs, int max_q_len, int H, int G, int hd,
                                          int vd, long long q_tok, long long q_head, long long o_tok,
                                          long long o_head, float scale, float softcap, int bias_rows,
-                                         int n_lookup, int window, hipStream_t stream) {
+                                         int n_lookup, int window, const float* gate,
+                                         long long gate_tok, hipStream_t stream) {
     if (n_seqs <= 0 || max_q_len <= 0) return 0;
     if (!gfa_scored_attention_mfma_takes(H, G, hd, vd, talk != nullptr) || n_seqs > 65535)
         return (int)hipErrorInvalidValue;
@@ -669,7 +675,7 @@ extern "C" int gfa_scored_attention_mfma(const void* q, const void* k_pages, con
     if (q_tok % 8 || q_head % 8 || o_tok % 2 || o_head % 2) return (int)hipErrorInvalidValue;
     if ((r1 == nullptr) != (r2 == nullptr)) return (int)hipErrorInvalidValue;
     SAShape s{H, G, hd, vd, q_tok, q_head, o_tok, o_head, table_stride, window, scale, softcap,
-              bias_rows, n_lookup, sink ? 1 : 0};
+              bias_rows, n_lookup, sink ? 1 : 0, gate, gate_tok};
 #define SAM_GO(DK, DVT, MAXT, SPLIT) return sam_launch<DK, DVT, MAXT, SPLIT>(q, k_pages, v_pages, q_start, \
         start_pos, table, temperature, bias, lookup, talk, r1, r2, out, n_seqs, max_q_len, s, stream)
     // one token per sequence and no mix: the waves of a workgroup share a tile's key blocks
@@ -862,15 +868,38 @@ extern "C" int gfa_whole_norm_store(const float* proj, int row_width, const floa
 // a row of proj is [q latent (q_rank) | kv latent (R) | key part to rotate (dr)].
 //   cq_out[n, :] = rmsnorm(q latent) * wq              (operand of the query's up projection)
 //   c = rmsnorm(kv latent) * wkv  -> the cache's key elements 0 .. R-1 and value elements 0 .. R-1
-//   rotated part: pairs (2i, 2i+1), i < rotary_dim / 2, turned by pos * freqs[i], the rest as
-//   it is -> the cache's key elements R .. R+dr-1
+//   rotated part: pairs (2i, 2i+1) (layout 0) or (i, i + rotary_dim / 2) (layout 1),
+//   i < rotary_dim / 2, turned by pos * freqs[i] with cos and sin times trig, the rest as it is
+//   -> the cache's key elements R .. R+dr-1
 // The cache has one kv head with keys of R + dr and values of R.  One workgroup per token.
+
+// The workgroup's threads turn the first `rot` of the dr elements at x and hand on all of them:
+// put(element, value).
+template <typename F>
+__device__ __forceinline__ void rotate_part(const float* __restrict__ x, int dr,
+                                            const float* __restrict__ freqs, int rot, int layout,
+                                            float trig, int pos, F put) {
+    const int half = rot >> 1;
+    for (int i = threadIdx.x; i < dr - half; i += blockDim.x) {
+        if (i >= half) {                               // behind the pairs: as it is
+            put(half + i, x[half + i]);
+            continue;
+        }
+        const int a = layout == 0 ? 2 * i : i, b = layout == 0 ? 2 * i + 1 : i + half;
+        const float u = x[a], v = x[b];
+        float sn, cs;
+        sincosf((float)pos * freqs[i], &sn, &cs);
+        put(a, (u * cs - v * sn) * trig);
+        put(b, (v * cs + u * sn) * trig);
+    }
+}
+
 template <typename T>
 __global__ __launch_bounds__(SA_THREADS) void latent_store_kernel(
         const float* __restrict__ proj, int row_width, int q_rank, int R, int dr,
         const float* __restrict__ wq, const float* __restrict__ wkv, float eps,
-        const float* __restrict__ freqs, int rotary_dim, T* __restrict__ cq_out,
-        T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ tok_seq,
+        const float* __restrict__ freqs, int rotary_dim, int layout, float trig,
+        T* __restrict__ cq_out, T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ tok_seq,
         const int* __restrict__ tok_pos, const int* __restrict__ table, int table_stride) {
     __shared__ float scratch[16];
     const int n = blockIdx.x;
@@ -896,37 +925,26 @@ __global__ __launch_bounds__(SA_THREADS) void latent_store_kernel(
         store_from_float(k_pages + key_elem(page, 0, slot, e, 1, hd), c);
         store_from_float(v_pages + value_elem(page, 0, e, slot, 1, R), c);
     }
-    const float* kr = kv + R;
-    for (int i = threadIdx.x; i < dr / 2; i += SA_THREADS) {
-        float u = kr[2 * i], v = kr[2 * i + 1];
-        if (2 * i < rotary_dim) {
-            float sn, cs;
-            sincosf((float)pos * freqs[i], &sn, &cs);
-            const float u2 = u * cs - v * sn, v2 = v * cs + u * sn;
-            u = u2;
-            v = v2;
-        }
-        store_from_float(k_pages + key_elem(page, 0, slot, R + 2 * i, 1, hd), u);
-        store_from_float(k_pages + key_elem(page, 0, slot, R + 2 * i + 1, 1, hd), v);
-    }
-    if ((dr & 1) && threadIdx.x == 0)
-        store_from_float(k_pages + key_elem(page, 0, slot, hd - 1, 1, hd), kr[dr - 1]);
+    rotate_part(kv + R, dr, freqs, rotary_dim, layout, trig, pos, [&](int e, float v) {
+        store_from_float(k_pages + key_elem(page, 0, slot, R + e, 1, hd), v);
+    });
 }
 
 extern "C" int gfa_latent_store(const float* proj, int row_width, int q_rank, int R, int dr,
                                 const float* wq, const float* wkv, float eps, const float* freqs,
-                                int rotary_dim, void* cq_out, void* k_pages, void* v_pages,
+                                int rotary_dim, int layout, float trig, void* cq_out, void* k_pages, void* v_pages,
                                 const int* tok_seq, const int* tok_pos, const int* table,
                                 int table_stride, int n_tokens, int is_bf16, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (rotary_dim % 2 || rotary_dim > dr) return (int)hipErrorInvalidValue;
+    if (rotary_dim < 0 || rotary_dim % 2 || rotary_dim > dr || (layout != 0 && layout != 1))
+        return (int)hipErrorInvalidValue;
     if (is_bf16)
         latent_store_kernel<bf16_t><<<n_tokens, SA_THREADS, 0, stream>>>(
-            proj, row_width, q_rank, R, dr, wq, wkv, eps, freqs, rotary_dim, (bf16_t*)cq_out,
+            proj, row_width, q_rank, R, dr, wq, wkv, eps, freqs, rotary_dim, layout, trig, (bf16_t*)cq_out,
             (bf16_t*)k_pages, (bf16_t*)v_pages, tok_seq, tok_pos, table, table_stride);
     else
         latent_store_kernel<float><<<n_tokens, SA_THREADS, 0, stream>>>(
-            proj, row_width, q_rank, R, dr, wq, wkv, eps, freqs, rotary_dim, (float*)cq_out,
+            proj, row_width, q_rank, R, dr, wq, wkv, eps, freqs, rotary_dim, layout, trig, (float*)cq_out,
             (float*)k_pages, (float*)v_pages, tok_seq, tok_pos, table, table_stride);
     return GFA_LAUNCH_RESULT();
 }
@@ -938,7 +956,8 @@ extern "C" int gfa_latent_store(const float* proj, int row_width, int q_rank, in
 // product fills.  A token's row starts q_stride floats after the one before.  grid (tokens, heads).
 template <typename T>
 __global__ void latent_query_kernel(const float* __restrict__ q, const float* __restrict__ freqs,
-                                    int rotary_dim, const int* __restrict__ tok_pos,
+                                    int rotary_dim, int layout, float trig,
+                                    const int* __restrict__ tok_pos,
                                     T* __restrict__ plain_out, T* __restrict__ full_out, int N, int H,
                                     int d, int dr, int R, long long q_stride) {
     const int n = blockIdx.x, h = blockIdx.y;
@@ -946,37 +965,24 @@ __global__ void latent_query_kernel(const float* __restrict__ q, const float* __
     T* plain = plain_out + ((size_t)h * N + n) * d;
     for (int e = threadIdx.x; e < d; e += blockDim.x) store_from_float(plain + e, row[e]);
     T* full = full_out + ((size_t)h * N + n) * (R + dr) + R;
-    const float* qr = row + d;
-    const int pos = tok_pos[n];
-    for (int i = threadIdx.x; i < dr / 2; i += blockDim.x) {
-        float u = qr[2 * i], v = qr[2 * i + 1];
-        if (2 * i < rotary_dim) {
-            float sn, cs;
-            sincosf((float)pos * freqs[i], &sn, &cs);
-            const float u2 = u * cs - v * sn, v2 = v * cs + u * sn;
-            u = u2;
-            v = v2;
-        }
-        store_from_float(full + 2 * i, u);
-        store_from_float(full + 2 * i + 1, v);
-    }
-    if ((dr & 1) && threadIdx.x == 0) store_from_float(full + dr - 1, qr[dr - 1]);
+    rotate_part(row + d, dr, freqs, rotary_dim, layout, trig, tok_pos[n],
+                [&](int e, float v) { store_from_float(full + e, v); });
 }
 
-extern "C" int gfa_latent_query(const float* q, const float* freqs, int rotary_dim,
-                                const int* tok_pos, void* plain_out, void* full_out, int n_tokens,
+extern "C" int gfa_latent_query(const float* q, const float* freqs, int rotary_dim, int layout,
+                                float trig, const int* tok_pos, void* plain_out, void* full_out, int n_tokens,
                                 int H, int d, int dr, int R, long long q_stride, int is_bf16,
                                 hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (H > 65535 || rotary_dim % 2 || rotary_dim > dr || q_stride < (long long)H * (d + dr))
+    if (H > 65535 || rotary_dim < 0 || rotary_dim % 2 || rotary_dim > dr || (layout != 0 && layout != 1) || q_stride < (long long)H * (d + dr))
         return (int)hipErrorInvalidValue;
     dim3 grid(n_tokens, H);
     if (is_bf16)
-        latent_query_kernel<bf16_t><<<grid, 64, 0, stream>>>(q, freqs, rotary_dim, tok_pos,
+        latent_query_kernel<bf16_t><<<grid, 64, 0, stream>>>(q, freqs, rotary_dim, layout, trig, tok_pos,
                                                              (bf16_t*)plain_out, (bf16_t*)full_out,
                                                              n_tokens, H, d, dr, R, q_stride);
     else
-        latent_query_kernel<float><<<grid, 64, 0, stream>>>(q, freqs, rotary_dim, tok_pos,
+        latent_query_kernel<float><<<grid, 64, 0, stream>>>(q, freqs, rotary_dim, layout, trig, tok_pos,
                                                             (float*)plain_out, (float*)full_out,
                                                             n_tokens, H, d, dr, R, q_stride);
     return GFA_LAUNCH_RESULT();

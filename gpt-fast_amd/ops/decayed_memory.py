@@ -99,13 +99,14 @@ def scan(proj: torch.Tensor, layout: RowLayout, decay: torch.Tensor, state: torc
 
 
 def row_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], proj: torch.Tensor, layout: RowLayout,
-                  eps: float, out_dtype: torch.dtype, groups: int = 1, gate: str = "sigmoid") -> torch.Tensor:
+                  eps: float, out_dtype: torch.dtype, groups: int = 1, gate: str = "sigmoid",
+                  gate_first: bool = False) -> torch.Tensor:
     """y[t, :] = o[t, :] / rms(o[t, :]) * weight * gate(g[t, :]) in ``out_dtype``, the root mean
     square taken over each of ``groups`` equal parts of the row (1: the whole row; the number
     of heads: every head by itself); o float32 [N, W]; ``weight`` float32 of W elements, or of
     fewer that divide W and are used again along the row (one weight shared by the heads), or
     None; the gate's pre-activations lie in proj at ``layout.g``; ``gate`` "sigmoid" or
-    "silu"."""
+    "silu".  ``gate_first``: o is multiplied by the gate before its parts are normed."""
     require_device(o, weight, proj)
     require_contiguous(o=o, weight=weight, proj=proj)
     n, width = o.shape
@@ -121,7 +122,8 @@ def row_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], proj: torch.T
     if gate not in ("sigmoid", "silu"):
         raise KernelError(f"row_norm_gate: gate '{gate}': sigmoid or silu")
     y = torch.empty((n, width), dtype=out_dtype, device=o.device)
-    check(library("decayed_memory").gfa_row_norm_gate(
+    lib = library("decayed_memory")
+    check((lib.gfa_gate_row_norm if gate_first else lib.gfa_row_norm_gate)(
         ptr(o), ptr(weight), _i(0 if weight is None else weight.numel()), ptr(proj), _i(layout.width),
         _i(layout.g), ptr(y), _i(int(out_dtype == torch.bfloat16)), _i(n), _i(width), _i(groups),
         _i(int(gate == "silu")), _f(eps), stream_handle()), "row_norm_gate")

@@ -1,6 +1,6 @@
-"""Python faces of the gated-delta-rule kernels of csrc/gated_delta.hip: the short causal
-convolutions with their tails, and the cell token by token.  Shape checks on the host, then
-the launch."""
+"""Python faces of the gated-delta-rule kernels of csrc/gated_delta.hip: the cell behind the short
+causal convolutions (ops/short_conv.py), token by token and a chunk of tokens at a time.  Shape
+checks on the host, then the launch."""
 import ctypes
 from dataclasses import dataclass
 
@@ -11,7 +11,6 @@ from .library import KernelError, check, library, ptr, require_contiguous, requi
 _i, _f, _sz = ctypes.c_int, ctypes.c_float, ctypes.c_size_t
 
 MAX_KEY_DIM = 512            # rows of S a workgroup's threads hold in registers
-MAX_TAPS = 16
 
 
 @dataclass(frozen=True)
@@ -52,32 +51,6 @@ def _check_step(proj, layout, state, q_start, slots, n_seqs):
         raise KernelError(f"gated delta: rows are {tuple(proj.shape)}, expected [N, {layout.width}]")
     if q_start.numel() < n_seqs + 1 or slots.numel() < n_seqs:
         raise KernelError("gated delta: q_start / slots are shorter than the batch")
-
-
-def short_conv(proj: torch.Tensor, layout: RowLayout, taps: torch.Tensor, state: torch.Tensor,
-               tail_offset: int, tok_seq, q_start, slots, n_seqs: int) -> torch.Tensor:
-    """silu of the causal convolution of the first ``layout.conv`` columns of proj over each
-    sequence's tokens, float32 [N, C]; taps float32 [C, K], the last column the current
-    token's.  ``state`` [slots, size] holds every sequence's last K - 1 inputs at
-    ``tail_offset`` ([K - 1, C], oldest first; zero for a new sequence) and is left holding the
-    step's."""
-    require_device(proj, taps, state, tok_seq, q_start, slots)
-    require_contiguous(proj=proj, taps=taps, state=state, tok_seq=tok_seq, q_start=q_start, slots=slots)
-    _check_step(proj, layout, state, q_start, slots, n_seqs)
-    C = layout.conv
-    if taps.dtype != torch.float32 or taps.dim() != 2 or taps.shape[0] != C or not 1 <= taps.shape[1] <= MAX_TAPS:
-        raise KernelError(f"short_conv: taps must be float32 [{C}, 1..{MAX_TAPS}]")
-    K = taps.shape[1]
-    if state.dim() != 2 or tail_offset < 0 or tail_offset + (K - 1) * C > state.shape[1]:
-        raise KernelError("short_conv: the tails do not fit the state")
-    if tok_seq.dtype != torch.int32 or tok_seq.numel() < proj.shape[0]:
-        raise KernelError("short_conv: tok_seq must be int32 and cover the batch")
-    y = torch.empty((proj.shape[0], C), dtype=torch.float32, device=proj.device)
-    check(library("gated_delta").gfa_short_conv(
-        ptr(proj), _i(layout.width), ptr(taps), _i(K), _i(C), ptr(state), _sz(state.stride(0)),
-        _sz(tail_offset), ptr(tok_seq), ptr(q_start), ptr(slots), ptr(y), _i(proj.shape[0]),
-        _i(n_seqs), stream_handle()), "short_conv")
-    return y
 
 
 CHUNKS_FROM_TOKENS = 16      # runs shorter than this go token by token

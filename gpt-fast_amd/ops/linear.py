@@ -228,6 +228,19 @@ def linear_into(x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, then_n
     return None
 
 
+def linear_terms(x: torch.Tensor, w: torch.Tensor):
+    """The product x W^T [M, N] for a reader that adds it to something itself: float32 or bfloat16
+    [M, N], or float32 [S, M, N] whose S slices are still to be added - whichever the fastest
+    product for these rows leaves."""
+    if x.dtype == torch.float32 or x.shape[0] <= SKINNY_MAX_ROWS:
+        return linear(x, w, out_dtype=torch.float32)
+    if x.shape[0] <= _wide().MAX_ROWS and w.shape[0] % 4 == 0 and _tiled_for(x.shape[0], w) is None \
+            and _sliced_is_faster(x.shape[0], w.shape[0], x.shape[1]):
+        return _wide().partial_sums(x, w)
+    rows = linear(x, w, may_stay_sliced=True)
+    return rows.part if isinstance(rows, SlicedRows) else rows
+
+
 def takes_chunked_rows(rows: int, dtype, w, then_norm, takes_halves: bool) -> bool:
     """:func:`linear_into` with these arguments runs the few-row kernel that also reads its x
     as ``gemm_bf16.ChunkedRows``."""

@@ -52,21 +52,22 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
               scale: float, *, window: int = 0, temperature: Optional[torch.Tensor] = None,
               softcap: float = 0.0, bias: Optional[torch.Tensor] = None,
               lookup: Optional[torch.Tensor] = None, talk: Optional[torch.Tensor] = None,
-              log_bias=None, sink: bool = False,
+              log_bias=None, sink: bool = False, gate: Optional[torch.Tensor] = None,
               head_major: bool = False, out: Optional[torch.Tensor] = None, step=None) -> torch.Tensor:
     """Each token's heads attend to the keys of its sequence's pages.  q is [N, H, hd], or
     [H, N, hd] if ``head_major`` (the result then lies the same way); k_pages
     [pages, G, 64, hd], v_pages [pages, G, vd, 64]; temperature float32 [H]; bias float32
     [rows, H] with lookup int32 [distances] (see :func:`distance_rows`); talk float32 [H, H];
     log_bias = (r1, r2), float32 [H] each: ``r1[h] ln(1 + r2[h] (i - j))`` is taken off the
-    score; sink: the softmax's denominator has one more term exp(0).
+    score; sink: the softmax's denominator has one more term exp(0); gate float32 [N, >= H], a
+    view of wider rows allowed: head h of token n is multiplied by ``sigmoid(gate[n, h])``.
     Returns [N, H, vd] (or [H, N, vd]) in q's type.  ``out`` may be a view with unit stride
     in its last dimension.  ``step`` = (q_start int32 [B + 1], start_pos int32 [B], B, longest
     run of new tokens) describes the same tokens sequence by sequence; with it, bfloat16 rows
     of sizes the matrix-core kernel takes go there."""
     r1, r2 = log_bias if log_bias is not None else (None, None)
     require_device(q, k_pages, v_pages, tok_seq, tok_pos, table, temperature, bias, lookup, talk, out,
-                   r1, r2)
+                   r1, r2, gate)
     require_contiguous(tok_seq=tok_seq, tok_pos=tok_pos, table=table, temperature=temperature,
                        bias=bias, lookup=lookup, talk=talk, r1=r1, r2=r2)
     if q.dim() != 3 or q.stride(2) != 1:
@@ -88,6 +89,10 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
                            ("r2", r2, H)):
         if t is not None and (t.dtype != torch.float32 or t.numel() != count):
             raise KernelError(f"scored attention: {name} must be float32 with {count} elements")
+    if gate is not None and (gate.dtype != torch.float32 or gate.dim() != 2 or gate.shape[0] != n
+                             or gate.shape[1] < H or (H > 1 and gate.stride(1) != 1)):
+        raise KernelError("scored attention: gate must be float32 [N, >= H] with unit stride along a row")
+    gate_tok = 0 if gate is None else gate.stride(0)
     rows = 0
     if bias is not None:
         if bias.dtype != torch.float32 or bias.dim() != 2 or bias.shape[1] != H or bias.shape[0] < 1:
@@ -123,7 +128,7 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
             _i(G), _i(hd), _i(vd),
             _ll(q.stride(tok)), _ll(q.stride(head)), _ll(out.stride(tok)), _ll(out.stride(head)),
             _f(scale), _f(softcap or 0.0), _i(rows), _i(0 if lookup is None else lookup.numel()),
-            _i(window or 0), stream_handle()), "scored_attention_mfma")
+            _i(window or 0), ptr(gate), _ll(gate_tok), stream_handle()), "scored_attention_mfma")
         return out
     check(lib.gfa_scored_attention(
         ptr(q), ptr(k_pages), ptr(v_pages), ptr(tok_seq), ptr(tok_pos), ptr(table),
@@ -132,7 +137,7 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
         _ll(q.stride(tok)),
         _ll(q.stride(head)), _ll(out.stride(tok)), _ll(out.stride(head)), _f(scale),
         _f(softcap or 0.0), _i(rows), _i(0 if lookup is None else lookup.numel()), _i(window or 0),
-        _i(_is_bf16(q)), stream_handle()), "scored_attention")
+        ptr(gate), _ll(gate_tok), _i(_is_bf16(q)), stream_handle()), "scored_attention")
     return out
 
 
@@ -182,10 +187,12 @@ def unit_heads_store(proj: torch.Tensor, bias: Optional[torch.Tensor], tok_seq, 
 
 def latent_store(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, q_weight, kv_weight,
                  eps: float, freqs: Optional[torch.Tensor], rotary_dim: int, tok_seq, tok_pos, table,
-                 k_pages, v_pages, out_dtype: torch.dtype) -> torch.Tensor:
+                 k_pages, v_pages, out_dtype: torch.dtype, layout: int = 0,
+                 trig_scale: float = 1.0) -> torch.Tensor:
     """The normed query latent [N, q_rank] in ``out_dtype`` from the float32 sums proj
     [N, >= q_rank + kv_rank + rot_dim]; the normed kv latent and the rotated key part go into
-    the cache (one kv head; keys of kv_rank + rot_dim, values of kv_rank; None: not)."""
+    the cache (one kv head; keys of kv_rank + rot_dim, values of kv_rank; None: not).  ``layout``
+    0: pairs (2i, 2i + 1), 1: pairs (i, i + rotary_dim / 2); cos and sin times ``trig_scale``."""
     require_device(proj, q_weight, kv_weight, freqs, tok_seq, tok_pos, table, k_pages, v_pages)
     require_contiguous(proj=proj, q_weight=q_weight, kv_weight=kv_weight, freqs=freqs,
                        tok_seq=tok_seq, tok_pos=tok_pos, table=table)
@@ -195,7 +202,7 @@ def latent_store(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, q_
     if (q_rank and (q_weight is None or q_weight.dtype != torch.float32 or q_weight.numel() != q_rank)) \
             or kv_weight.dtype != torch.float32 or kv_weight.numel() != kv_rank:
         raise KernelError("latent_store: the norm weights must be float32 of the latents' sizes")
-    if rotary_dim % 2 or rotary_dim > rot_dim:
+    if rotary_dim % 2 or not 0 <= rotary_dim <= rot_dim or layout not in (0, 1):
         raise KernelError(f"latent_store: rotary_dim {rotary_dim} must be even and at most {rot_dim}")
     if rotary_dim and (freqs is None or freqs.dtype != torch.float32 or freqs.numel() != rotary_dim // 2):
         raise KernelError(f"latent_store: {rotary_dim // 2} float32 frequencies are needed")
@@ -208,7 +215,7 @@ def latent_store(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, q_
     cq = torch.empty((n, q_rank), dtype=out_dtype, device=proj.device)
     check(library("scored_attention").gfa_latent_store(
         ptr(proj), _i(proj.shape[1]), _i(q_rank), _i(kv_rank), _i(rot_dim), ptr(q_weight),
-        ptr(kv_weight), _f(eps), ptr(freqs), _i(rotary_dim), ptr(cq), ptr(k_pages), ptr(v_pages),
+        ptr(kv_weight), _f(eps), ptr(freqs), _i(rotary_dim), _i(layout), _f(trig_scale), ptr(cq), ptr(k_pages), ptr(v_pages),
         ptr(tok_seq), ptr(tok_pos), ptr(table), _i(table.shape[1]), _i(n),
         _i(int(out_dtype == torch.bfloat16)), stream_handle()), "latent_store")
     return cq
@@ -259,10 +266,12 @@ def whole_norm_store(proj: torch.Tensor, bias: Optional[torch.Tensor], q_weight,
 
 
 def latent_query(q: torch.Tensor, freqs: Optional[torch.Tensor], rotary_dim: int, tok_pos,
-                 n_heads: int, head_dim: int, rot_dim: int, kv_rank: int, out_dtype: torch.dtype):
+                 n_heads: int, head_dim: int, rot_dim: int, kv_rank: int, out_dtype: torch.dtype,
+                 layout: int = 0, trig_scale: float = 1.0):
     """From the float32 sums q [N, H (d + dr)] of the query's up projection: the plain parts
     head by head, [H, N, d], and a tensor [H, N, kv_rank + dr] whose last dr elements hold the
-    rotated parts (the first kv_rank are left for the product with the keys' up projection)."""
+    rotated parts (the first kv_rank are left for the product with the keys' up projection);
+    ``layout`` and ``trig_scale`` as in :func:`latent_store`."""
     require_device(q, freqs, tok_pos)
     require_contiguous(freqs=freqs, tok_pos=tok_pos)
     n = q.shape[0]
@@ -270,7 +279,7 @@ def latent_query(q: torch.Tensor, freqs: Optional[torch.Tensor], rotary_dim: int
             or q.stride(1) != 1:
         raise KernelError(f"latent_query: q must be float32 [N, {n_heads * (head_dim + rot_dim)}] "
                           f"with unit stride along a row (a view of wider rows is allowed)")
-    if rotary_dim % 2 or rotary_dim > rot_dim:
+    if rotary_dim % 2 or not 0 <= rotary_dim <= rot_dim or layout not in (0, 1):
         raise KernelError(f"latent_query: rotary_dim {rotary_dim} must be even and at most {rot_dim}")
     if rotary_dim and (freqs is None or freqs.dtype != torch.float32 or freqs.numel() != rotary_dim // 2):
         raise KernelError(f"latent_query: {rotary_dim // 2} float32 frequencies are needed")
@@ -279,7 +288,7 @@ def latent_query(q: torch.Tensor, freqs: Optional[torch.Tensor], rotary_dim: int
     plain = torch.empty((n_heads, n, head_dim), dtype=out_dtype, device=q.device)
     full = torch.empty((n_heads, n, kv_rank + rot_dim), dtype=out_dtype, device=q.device)
     check(library("scored_attention").gfa_latent_query(
-        ptr(q), ptr(freqs), _i(rotary_dim), ptr(tok_pos), ptr(plain), ptr(full), _i(n), _i(n_heads),
+        ptr(q), ptr(freqs), _i(rotary_dim), _i(layout), _f(trig_scale), ptr(tok_pos), ptr(plain), ptr(full), _i(n), _i(n_heads),
         _i(head_dim), _i(rot_dim), _i(kv_rank), _ll(q.stride(0)),
         _i(int(out_dtype == torch.bfloat16)), stream_handle()), "latent_query")
     return plain, full

@@ -4,6 +4,7 @@ import torch
 from ..config.spec import LayerSpec
 from ..ops import kernels as K
 from ..ops import linear as L
+from ..ops import streams as ST
 from .base import (FEED_FORWARDS, MIXERS, NORMS, Param, Part, ResidualStream, Runtime, check_bound,
                    register_block)
 
@@ -369,6 +370,117 @@ class PostNormBlock(PreNormBlock):
             stream.tensor                    # a caller with a plain tensor gets the sums now
 
 
+class StreamWeights(Part):
+    """The stored numbers with which one sublayer reads and writes S residual streams: ``in [S]``,
+    ``out [S]``, ``mix [S, S]`` (from, to)."""
+
+    replayable = True
+
+    def __init__(self, streams: int, runtime: Runtime):
+        self.streams = streams
+        self.w_in = self.w_out = self.mix = None
+
+    def parameters(self):
+        S = self.streams
+        return {"in": Param((S,), role="vector", init="share"),
+                "out": Param((S,), role="vector", init="norm"),
+                "mix": Param((S, S), role="vector", init="near_identity")}
+
+    def bind(self, tensors):
+        check_bound("StreamWeights", self.parameters(), tensors)
+        self.w_in, self.w_out, self.mix = (tensors[k].to(torch.float32).contiguous()
+                                           for k in ("in", "out", "mix"))
+
+
+class StreamRead:
+    """What reads several streams: ``norm(sum_s in[s] x_s)``.  It stands where a norm of one stream
+    would (``ResidualStream.normed``); ``stream_form()`` tells the kernel that completes the
+    streams how to make its rows on the way."""
+
+    def __init__(self, norm, runtime: Runtime, weights: StreamWeights = None, streams: int = 0):
+        if not hasattr(norm, "row_and_column_form"):
+            raise TypeError("streams are read through a norm with row_and_column_form() (kind 'rms')")
+        self.norm, self.rt, self.weights = norm, runtime, weights
+        # without weights: the plain sum of the streams
+        self.ones = None if weights is not None else torch.ones(streams, dtype=torch.float32,
+                                                                device=runtime.device)
+
+    def stream_form(self):
+        weight, eps = self.norm.row_and_column_form()
+        return self.ones if self.weights is None else self.weights.w_in, weight, eps
+
+    def forward(self, streams, rows=None):
+        return ST.read(streams, *self.stream_form(), self.rt.dtype, rows=rows)
+
+
+class HyperConnectedBlock(PreNormBlock):
+    """Hyper-connections: the residual is S streams, float32 ``[N, S, D]``; each sublayer reads
+    ``norm(sum_s in[s] x_s)``, and its result y moves all streams at once, from the old ones:
+    ``x_t <- sum_s mix[s, t] x_s + out[t] y``.  One kernel does that move and, where it is known
+    which read comes next (the block's own second sublayer's, the next layer's, the final
+    norm's), makes that reader's rows in the same pass; the last move of a sublayer is therefore
+    put off until the streams are read next.  A sublayer that offers ``forward_last(x, batch[,
+    entry]) -> (operand, matrix)`` leaves its last product to the block, whose result may then
+    be partial sums or bfloat16 rows, added on the kernel's way; else ``forward_rows``."""
+
+    takes_stream = True
+    takes_prepared = False
+
+    def __init__(self, spec: LayerSpec, runtime: Runtime):
+        super().__init__(spec, runtime)
+        if not spec.streams or not 1 <= spec.streams <= ST.MAX_STREAMS:
+            raise ValueError(f"a hyper_connected block works on 1..{ST.MAX_STREAMS} streams, not {spec.streams}")
+        self.rt = runtime
+        self.mixer_streams = StreamWeights(spec.streams, runtime)
+        self.mixer_read = StreamRead(self.mixer_norm, runtime, self.mixer_streams)
+        self.feed_forward_streams = self.feed_forward_read = None
+        if spec.feed_forward is not None:
+            self.feed_forward_streams = StreamWeights(spec.streams, runtime)
+            self.feed_forward_read = StreamRead(self.feed_forward_norm, runtime, self.feed_forward_streams)
+
+    # its own kernels beside those of its parts
+    libraries = ("streams",)
+
+    def children(self):
+        out = super().children()
+        out[self.spec.mixer_streams_name] = self.mixer_streams
+        if self.feed_forward is not None:
+            out[self.spec.feed_forward_streams_name] = self.feed_forward_streams
+        return out
+
+    def _result(self, part, args, streams):
+        """A sublayer's result alone, in whatever form the joining kernel takes."""
+        if hasattr(part, "forward_last"):
+            return L.linear_terms(*part.forward_last(*args))
+        if hasattr(part, "forward_rows"):
+            return part.forward_rows(*args)
+        y = torch.zeros_like(streams[:, 0])
+        part.forward(*args, y)
+        return y
+
+    def _join(self, streams, y, weights, next_read):
+        """Move the streams by y; the rows of ``next_read`` over the new ones, or None."""
+        form = getattr(next_read, "stream_form", None)
+        if form is None:
+            ST.join(streams, y, weights.mix, weights.w_out)
+            return None if next_read is None else next_read.forward(streams)
+        w_in, norm_weight, eps = form()
+        return ST.join(streams, y, weights.mix, weights.w_out, w_in, norm_weight, eps, self.rt.dtype)
+
+    def forward(self, residual, batch, entry):
+        stream = residual if isinstance(residual, ResidualStream) else ResidualStream(residual)
+        x = stream.normed(self.mixer_read)
+        y = self._result(self.mixer, (x, batch, entry), stream.tensor)
+        stream.defer(lambda X, then, halves: self._join(X, y, self.mixer_streams, then))
+        if self.feed_forward is not None:
+            h = stream.normed(self.feed_forward_read)
+            y2 = self._result(self.feed_forward, (h, batch), stream.tensor)
+            stream.defer(lambda X, then, halves: self._join(X, y2, self.feed_forward_streams, then))
+        if stream is not residual:
+            stream.tensor                    # a caller with a plain tensor gets the sums now
+
+
 register_block("pre_norm", PreNormBlock)
+register_block("hyper_connected", HyperConnectedBlock)
 register_block("post_norm", PostNormBlock)
 register_block("sandwich_norm", SandwichNormBlock)

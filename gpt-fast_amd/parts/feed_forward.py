@@ -95,6 +95,10 @@ class DenseFeedForward(Part):
         add_late(residual, lambda rows, then_norm, takes_halves: L.linear_into(
             self._inner(x), self.w_down, rows, then_norm, takes_halves))
 
+    def forward_last(self, x, batch):
+        """The operand and the matrix of the last product, which the block runs."""
+        return self._inner(x), self.w_down
+
     def forward_rows(self, x, batch):
         """The feed-forward's output alone: the second product's float32 sums."""
         return L.linear(self._inner(x), self.w_down, out_dtype=torch.float32)

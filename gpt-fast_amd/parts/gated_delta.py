@@ -8,6 +8,7 @@ from ..config.spec import GatedDeltaSpec
 from ..ops import decayed_memory as DM
 from ..ops import gated_delta as GD
 from ..ops import linear as L
+from ..ops import short_conv as SC
 from .base import Param, Part, Runtime, add_late, check_bound, register_mixer
 
 
@@ -27,16 +28,16 @@ class GatedDelta(Part):
     engine's type."""
 
     replayable = True
-    libraries = ("gated_delta", "decayed_memory")
+    libraries = ("gated_delta", "short_conv", "decayed_memory")
     defers_sum = True              # ``residual`` may be a parts.base.ResidualStream
 
     def __init__(self, spec: GatedDeltaSpec, runtime: Runtime):
         s = spec
         if s.n_heads % s.n_kv_heads:
             raise ValueError(f"gated delta: {s.n_heads} heads do not divide into {s.n_kv_heads} key heads")
-        if s.key_dim > GD.MAX_KEY_DIM or not 1 <= s.conv_taps <= GD.MAX_TAPS:
+        if s.key_dim > GD.MAX_KEY_DIM or not 1 <= s.conv_taps <= SC.MAX_TAPS:
             raise ValueError(f"gated delta: key_dim {s.key_dim} (up to {GD.MAX_KEY_DIM}), "
-                             f"{s.conv_taps} taps (1..{GD.MAX_TAPS})")
+                             f"{s.conv_taps} taps (1..{SC.MAX_TAPS})")
         self.spec = spec
         self.rt = runtime
         rows = GD.RowLayout.fused(s.n_heads, s.n_kv_heads, s.key_dim, s.value_dim)
@@ -76,8 +77,8 @@ class GatedDelta(Part):
     def _gated(self, x, batch, entry):
         s = self.spec
         proj = L.linear(x, self.w_in, out_dtype=torch.float32)
-        conv = GD.short_conv(proj, self.rows, self.taps, entry.state, self.tail_offset, batch.tok_seq,
-                             batch.q_start, batch.slots, batch.n_seqs)
+        conv = SC.short_conv(proj, self.taps, entry.state, self.tail_offset, batch.tok_seq,
+                             batch.q_start, batch.slots, batch.n_seqs, max_q_len=batch.max_q_len)
         o = GD.cell(conv, proj, self.rows, self.A_log, self.dt_bias, entry.state, batch.q_start,
                     batch.slots, batch.n_seqs, batch.max_q_len, s.n_heads, s.n_kv_heads, s.key_dim,
                     s.value_dim, s.key_dim ** -0.5, s.unit_eps)

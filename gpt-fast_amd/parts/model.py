@@ -6,8 +6,10 @@ import torch
 from ..config.spec import ModelPlan
 from ..ops import kernels as K
 from ..ops import linear as L
+from ..ops import streams as ST
 from .base import (BLOCKS, INPUT_ADDS, NORMS, POSITIONS, STREAM_STEPS, Param, ResidualStream, Runtime,
                    check_bound)
+from .block import StreamRead
 
 
 class DecoderModel:
@@ -26,6 +28,9 @@ class DecoderModel:
         self.rt = runtime
         self.blocks = [BLOCKS.build(_Arranged(layer), runtime) for layer in plan.layers]
         self.final_norm = NORMS.build(plan.final_norm, runtime)
+        # what reads the stream last: the final norm, over the sum of the streams if there are several
+        self.final_read = self.final_norm if plan.streams is None else \
+            StreamRead(self.final_norm, runtime, streams=plan.streams)
         self.input_position = None
         if plan.input_position is not None:
             self.input_position = POSITIONS.build(plan.input_position, runtime)
@@ -43,8 +48,8 @@ class DecoderModel:
             if spec is not None and spec not in self.enter_steps:
                 self.enter_steps[spec] = STREAM_STEPS.build(spec, runtime)
         self.embedding = self.head = None
-        # ``tap(n, rows)`` is called with the float32 stream [N, D] after run n of the order
-        # (tracing, tests); None: nothing is called
+        # ``tap(n, rows)`` is called with the float32 stream [N, D] (the sum of several) after run n of
+        # the order (tracing, tests); None: nothing is called
         self.tap = None
 
     # ------------------------------------------------------------------ parameters
@@ -198,6 +203,8 @@ class DecoderModel:
             part.add_to_stream(residual, batch, cache.entries[len(plan.order) + i])
         if self.input_position is not None:
             self.input_position.add_to_stream(residual, batch)
+        if plan.streams is not None:
+            residual = ST.spread(residual, plan.streams)
         stream = ResidualStream(residual)
         # the embedded rows, for steps that mix them into the stream again; a copy where a
         # block may have changed the stream (in place) before the first such step
@@ -213,7 +220,7 @@ class DecoderModel:
             block.forward(stream if getattr(block, "takes_stream", False) else stream.tensor,
                           batch, cache.entries[n])
             if self.tap is not None:
-                self.tap(n, stream.tensor)
+                self.tap(n, stream.tensor if plan.streams is None else stream.tensor.sum(1))
         if batch.n_want == 0:
             stream.tensor
             return torch.empty((0, self.plan.vocab_size), dtype=torch.float32,
@@ -221,7 +228,7 @@ class DecoderModel:
         # the head takes plain rows (no reader named): with its many columns the halves of a
         # norm cost more than the norm kernel they save
         every = getattr(batch, "every_row_wanted", False)
-        x = stream.normed(self.final_norm, rows=None if every else batch.want_rows)   # model.py:144
+        x = stream.normed(self.final_read, rows=None if every else batch.want_rows)   # model.py:144
         logits = L.linear(x, self.head, out_dtype=torch.float32)          # model.py:145
         if plan.logit_scale is not None or plan.logit_softcap is not None:
             K.scale_cap(logits, 1.0 if plan.logit_scale is None else plan.logit_scale,

@@ -29,6 +29,11 @@ INITS = {
     "positive": lambda t, std, norm_std: t.mul_(norm_std).add_(1.0).abs_(),   # |1 + N(0, norm_std)|
     # a square matrix near the identity (weights that mix heads)
     "head_mix": lambda t, std, norm_std: t.mul_(norm_std).add_(torch.eye(t.shape[0], device=t.device)),
+    # the same with entries whose spread shrinks with the size (a mix applied layer after layer)
+    "near_identity": lambda t, std, norm_std: t.mul_(norm_std / t.shape[0]).add_(
+        torch.eye(t.shape[0], device=t.device)),
+    # around an equal share each (weights of a sum of so many rows)
+    "share": lambda t, std, norm_std: t.mul_(norm_std).add_(1.0).div_(t.numel()),
 }
 
 

@@ -300,6 +300,7 @@ def test_the_convolutions_tails_and_the_delta_rule_with_carried_state(H, G, dk, 
     tokens, shorter than the taps); state and tails travel from step to step; token by token,
     and a chunk of 32 or of 64 tokens at a time."""
     from gpt_fast_amd.ops import gated_delta as GD
+    from gpt_fast_amd.ops import short_conv as SC
     g = torch.Generator().manual_seed(H * 31 + dk)
     layout = GD.RowLayout.fused(H, G, dk, dv)
     C = layout.conv
@@ -325,7 +326,8 @@ def test_the_convolutions_tails_and_the_delta_rule_with_carried_state(H, G, dk, 
         tok_seq = _ints([i for i, n in enumerate(take) for _ in range(n)])
         sl = _ints([slots[b] for b in live])
         rows_dev = _f32(rows)
-        conv = GD.short_conv(rows_dev, layout, _f32(taps), state, tail_off, tok_seq, q_start, sl, len(live))
+        conv = SC.short_conv(rows_dev, _f32(taps), state, tail_off, tok_seq, q_start, sl, len(live),
+                             max_q_len=max(take))
         o = GD.scan(conv, rows_dev, layout, _f32(A_log), _f32(dt_bias), state, q_start, sl, len(live),
                     H, G, dk, dv, dk ** -0.5, 1e-6, chunked=bool(chunked), max_q_len=chunked)
         at = 0
