@@ -133,7 +133,8 @@ extern "C" int gfa_state_space_scan(const float* conv, int conv_width, const flo
 // --------------------------------------------------------------------------------------
 // The same cell for runs of many tokens, a chunk of SC_L (32 or 64) tokens at a time.  With S0 the
 // state at the chunk's start, t, s = 0, 1, ... the chunk's tokens, L_t = sum_{r<=t} ln a_r and
-// e(t, s) = exp(L_t - L_s) <= 1 for s <= t, the recurrence written out is
+// e(t, s) = exp(L_t - L_s) <= 1 for s <= t (L in double: one fast decay must not cost the slow ones
+// behind it their digits), the recurrence written out is
 //     P[t][s] = (C_t . B_s) e(t, s) dt_s  for s <= t
 //     y_t = exp(L_t) S0^T C_t + sum_s P[t][s] x_s + D x_t
 //     S_end = exp(L_end) S0 + sum_s e(end, s) dt_s B_s x_s^T
@@ -175,8 +176,8 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
     float* St = Bs + SC_L * KS;                  // [SC_COLS][KS]  S transposed
     float* Xt = St + SC_COLS * KS;               // [SC_COLS][TS]  x transposed
     float* Ps = Xt + SC_COLS * TS;               // [SC_L][TS]
-    float* run = Ps + SC_L * TS;                 // [SC_L]  L_t
-    float* dts = run + SC_L;                     // [SC_L]  dt_t, 0 beyond the chunk's end
+    double* run = (double*)(Ps + SC_L * TS);     // [SC_L]  L_t
+    float* dts = (float*)(run + SC_L);           // [SC_L]  dt_t, 0 beyond the chunk's end
     float* wl = dts + SC_L;                      // [SC_L]  e(end, s) dt_s, 0 beyond the chunk's end
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int li = lane & 15, lg = lane >> 4;
@@ -253,17 +254,17 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
             // the first wave: step sizes, and the running sum of the log decays over its lanes
             const bool mine = tid < Lc;
             const float dt = mine ? ss_softplus(rd + bias) : 0.f;
-            float sum = -rate * dt;
+            double sum = -rate * dt;
 #pragma unroll
             for (int o = 1; o < SC_L; o <<= 1) {
-                const float up = __shfl_up(sum, o, 64);
+                const double up = __shfl_up(sum, o, 64);
                 if (tid >= o) sum += up;
             }
-            const float last = __shfl(sum, SC_L - 1, 64);
+            const double last = __shfl(sum, SC_L - 1, 64);
             if (tid < SC_L) {
                 run[tid] = sum;
                 dts[tid] = dt;
-                wl[tid] = mine ? expf(last - sum) * dt : 0.f;
+                wl[tid] = mine ? expf((float)(last - sum)) * dt : 0.f;
             }
         }
         if (c0 + SC_L < t1) fetch(c0 + SC_L);
@@ -284,7 +285,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int t = ti * 16 + lg * 4 + r;
-                Ps[t * TS + ss] = ss <= t ? acc[r] * expf(run[t] - run[ss]) * dts[ss] : 0.f;
+                Ps[t * TS + ss] = ss <= t ? acc[r] * expf((float)(run[t] - run[ss])) * dts[ss] : 0.f;
             }
         }
         // the state's share of y for the workgroup's columns: exp(L_t) (C S0)
@@ -297,7 +298,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
             for (int d0 = 0; d0 < Np; d0 += 16)
                 num = sc_mfma4(*(const float4*)(ca + d0), *(const float4*)(sb + d0), num);
 #pragma unroll
-            for (int r = 0; r < 4; ++r) num[r] *= expf(run[oti * 16 + lg * 4 + r]);
+            for (int r = 0; r < 4; ++r) num[r] *= expf((float)run[oti * 16 + lg * 4 + r]);
         }
         __syncthreads();                         // Ps is whole, St has been read by every wave
         {
@@ -316,7 +317,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
         // the state after the chunk's last token, transposed: S^T = exp(L_end) S^T + (x w)^T B, a
         // wave's tiles of 16 columns of x by 16 rows of S in turn
         {
-            const float aL = expf(run[SC_L - 1]);
+            const float aL = expf((float)run[SC_L - 1]);
             for (int tile = wave; tile < (Np / 16) * 2; tile += NW) {
                 const int di = tile >> 1, ci = tile & 1;
                 sc_floatx4_t acc;
@@ -345,7 +346,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
 }
 
 static int sc_lds_bytes(int N, int L) {
-    return (int)sizeof(float) * ((2 * L + SC_COLS) * sc_row_stride(N) + (SC_COLS + L) * (L + 4) + 3 * L);
+    return (int)sizeof(float) * ((2 * L + SC_COLS) * sc_row_stride(N) + (SC_COLS + L) * (L + 4) + 4 * L);
 }
 
 static int sc_lds_limit() {

@@ -211,3 +211,10 @@ def forward(w, cfg, tokens, taps=None):
     logits = rms_norm(X.sum(0), w["final.norm"], eps) @ w["embed"].T
     cap = cfg.get("logit_softcap")
     return logits if not cap else cap * torch.tanh(logits / cap)
+
+
+def greedy_generate(w, cfg, prompt, max_new_tokens):
+    tokens = list(prompt)
+    for _ in range(max_new_tokens):
+        tokens.append(int(forward(w, cfg, tokens)[-1].argmax()))
+    return tokens[len(prompt):]

@@ -1,0 +1,781 @@
+"""Bikadra on the GPU against the plain float64 implementation of tests/plain_bikadra.py: each
+mechanism's kernels alone (the streams' read and move in every form, the short convolution with
+its bias and tails, the state-space cell with carried state, the gate before the norm, the
+latents with half-split rotation, the attention's gate per head and a key that stands out), the
+block with parts of every kind, whole prompts with the streams' sum after every run, prompts in
+portions, token-by-token decoding, unequal batches, slots and pages that come back, far keys at
+page borders, state that lasts for hundreds of tokens, long decoding, and greedy generation
+through the library's generation loop, command line and trace replay."""
+import os
+
+import pytest
+import torch
+
+import plain_bikadra as P
+import util
+from bikadra_cases import CASES, make_folder, random_case, write_model
+from util import TOL_BF16, rel_err
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+F = torch.float64
+# float32 engine against float64 over a few hundred tokens and several norms
+TOL_F32_LONG = 1e-4
+
+
+def row_errors(got, want):
+    """Per row: root mean square of the difference over that of all of ``want``."""
+    got, want = got.double().cpu(), want.double().cpu()
+    return (got - want).pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+
+
+def close(got, want, dtype, tol):
+    """float32: the largest difference.  bfloat16: single positions of these small random models
+    answer a rounding of the embedded rows alone with a difference of 0.1 to 0.6 (a normed part
+    that is nearly zero), so the typical row is held to the tolerance and all but one in fifty
+    (at least one) to a bound that a wrong key, a lost state or a missing term, which touch most
+    rows, would break; the float32 engine is the sharp test."""
+    if dtype == "float32":
+        return rel_err(got, want) < tol
+    e = row_errors(got, want).sort().values
+    rest = e[:max(1, e.numel() - max(1, e.numel() // 50))]
+    return float(rest.max()) < 0.25 and float(e.median()) < 1.5 * TOL_BF16
+
+
+def _engine(folder, dtype, **kw):
+    import gpt_fast_amd as gfa
+    kw.setdefault("max_tokens", 4096)
+    return gfa.Engine.from_folder(folder, dtype=dtype, device=DEV, **kw)
+
+
+def _steps(eng, toks, cuts):
+    """Feed ``toks`` as one sequence in portions that end at ``cuts``; logits of every token."""
+    import gpt_fast_amd as gfa
+    slot = eng.start_sequence()
+    out, lo = [], 0
+    for hi in list(cuts) + [len(toks)]:
+        if hi <= lo:
+            continue
+        out.append(eng.step([gfa.Entry(slot, toks[lo:hi], want=list(range(hi - lo)))]).cpu())
+        lo = hi
+    eng.end_sequence(slot)
+    return torch.cat(out)
+
+
+def _ints(values):
+    return torch.tensor(values, dtype=torch.int32, device=DEV)
+
+
+def _f32(t):
+    return t.to(torch.float32).to(DEV).contiguous()
+
+
+def _table_and_positions(lens, starts):
+    """Pages handed out in reverse; the step's token maps."""
+    total = [s + l for s, l in zip(starts, lens)]
+    n_pages = sum((t + 63) // 64 for t in total)
+    order, tables, at = list(range(n_pages))[::-1], [], 0
+    for t in total:
+        n = (t + 63) // 64
+        tables.append(order[at:at + n])
+        at += n
+    widest = max(len(t) for t in tables)
+    table = _ints([t + [-1] * (widest - len(t)) for t in tables])
+    tok_seq = _ints([b for b, l in enumerate(lens) for _ in range(l)])
+    pos = [s + i for s, l in zip(starts, lens) for i in range(l)]
+    return n_pages, tables, table, tok_seq, _ints(pos), pos
+
+
+# --------------------------------------------------------------------------- streams
+@pytest.mark.parametrize("S", [1, 2, 3, 4, 5, 16])
+@pytest.mark.parametrize("dim", [50, 96, 1030, 4096, 8200])
+def test_streams_are_spread_read_and_moved(S, dim):
+    from gpt_fast_amd.ops import streams as ST
+    g = torch.Generator().manual_seed(S * 10000 + dim)
+    n = 5
+    X = torch.randn(S, n, dim, generator=g, dtype=F)
+    y = torch.randn(n, dim, generator=g, dtype=F) * 2
+    a, b, nxt = (torch.randn(S, generator=g, dtype=F) for _ in range(3))
+    mix = torch.randn(S, S, generator=g, dtype=F)
+    w = torch.rand(dim, generator=g, dtype=F) + 0.5
+    eps = 1e-3
+    dev = _f32(X.permute(1, 0, 2))
+    assert torch.equal(ST.spread(dev[:, 0].contiguous(), S), dev[:, :1].expand(n, S, dim))
+    for dtype, tol in ((torch.float32, 1e-5), (torch.bfloat16, 1e-2)):
+        want = P.rms_norm(P.stream_read(X, a), w, eps)
+        assert rel_err(ST.read(dev, _f32(a), _f32(w), eps, dtype), want) < tol
+        assert rel_err(ST.read(dev, _f32(a), _f32(w), eps, dtype, rows=_ints([4, 0, 4])), want[[4, 0, 4]]) < tol
+        # y as float32 rows, as bfloat16 rows, as three partial sums
+        parts = torch.randn(2, n, dim, generator=g, dtype=F)
+        forms = [(y, _f32(y)), (y.bfloat16().to(F), y.bfloat16().to(DEV)),
+                 (y, _f32(torch.stack([y - parts[0] - parts[1], parts[0], parts[1]])))]
+        for value, form in forms:
+            new = P.stream_write(X, mix, b, value)
+            moved = dev.clone()
+            out = ST.join(moved, form, _f32(mix), _f32(b), _f32(nxt), _f32(w), eps, dtype)
+            assert rel_err(moved.permute(1, 0, 2), new) < 1e-5
+            assert rel_err(out, P.rms_norm(P.stream_read(new, nxt), w, eps)) < tol
+            again = dev.clone()
+            assert ST.join(again, form, _f32(mix), _f32(b)) is None
+            assert torch.equal(again, moved)
+
+
+@pytest.mark.parametrize("rows", [1, 16, 17, 64, 65, 300])
+def test_a_product_s_terms_add_up_to_the_product(rows):
+    from gpt_fast_amd.ops import linear as L
+    torch.manual_seed(rows)
+    for N, K in ((96, 40), (256, 4096), (100, 600), (4096, 1024)):
+        for dtype, tol in ((torch.float32, 1e-5), (torch.bfloat16, 1e-2)):
+            x, w = torch.randn(rows, K, device=DEV).to(dtype), torch.randn(N, K, device=DEV).to(dtype)
+            got = L.linear_terms(x, w)
+            assert got.dtype in (torch.float32, dtype)
+            got = got.double().cpu()
+            assert rel_err(got.sum(0) if got.dim() == 3 else got, x.double().cpu() @ w.double().cpu().T) < tol
+
+
+@pytest.mark.parametrize("dtype,tol", [("float32", 1e-5), ("bfloat16", 2e-2)])
+def test_the_block_with_parts_that_offer_less(dtype, tol):
+    """A mixer that only adds into the stream, a feed-forward that only adds (gated), and one
+    that leaves its last product to the block; the block called with the plain tensor."""
+    import gpt_fast_amd as gfa
+    from gpt_fast_amd.config.spec import DenseFeedForwardSpec, GatedFeedForwardSpec, LayerSpec, NormSpec
+    from gpt_fast_amd.parts.base import BLOCKS, Runtime
+    from gpt_fast_amd.parts.model import _Arranged
+
+    class Tripling:
+        kind = "tripling_for_a_test"
+
+    class TriplingMixer:
+        def __init__(self, spec, runtime):
+            pass
+
+        def parameters(self):
+            return {}
+
+        def bind(self, tensors):
+            pass
+
+        def cache_need(self):
+            return None
+
+        def forward(self, x, batch, entry, residual):
+            residual += 3.0 * x.float()
+    gfa.register_mixer("tripling_for_a_test", TriplingMixer)
+    rt = Runtime(torch.float32 if dtype == "float32" else torch.bfloat16, DEV)
+    D, H, S = 72, 136, 3
+    for ff in (GatedFeedForwardSpec(D, H, "silu"), DenseFeedForwardSpec(D, H, "gelu_tanh"), None):
+        layer = LayerSpec(name="l", arrangement="hyper_connected", streams=S, mixer=Tripling(),
+                          mixer_norm=NormSpec(D, 1e-5), feed_forward=ff,
+                          feed_forward_norm=None if ff is None else NormSpec(D, 1e-5))
+        block = BLOCKS.build(_Arranged(layer), rt)
+        torch.manual_seed(8)
+        t = {}
+        for name, p in block.parameters().items():
+            scale = 0.3 if p.role == "matrix" else 1.0
+            t[name] = (torch.randn(p.shape, device=DEV) * scale).to(rt.dtype if p.role == "matrix" else torch.float32)
+        block.bind(t)
+        d = {k: v.double().cpu() for k, v in t.items()}
+        for rows in (2, 40, 130):
+            X = torch.randn(rows, S, D, device=DEV)
+            want = X.double().cpu().permute(1, 0, 2)
+            block.forward(X, None, None)
+            y = 3.0 * P.rms_norm(P.stream_read(want, d["mixer_streams.in"]), d["mixer_norm.weight"], 1e-5)
+            want = P.stream_write(want, d["mixer_streams.mix"], d["mixer_streams.out"], y)
+            if ff is not None:
+                h = P.rms_norm(P.stream_read(want, d["feed_forward_streams.in"]), d["feed_forward_norm.weight"], 1e-5)
+                if ff.kind == "gated":
+                    gu = h @ d["feed_forward.w13"].T
+                    y = (P.silu(gu[:, :H]) * gu[:, H:]) @ d["feed_forward.w2"].T
+                else:
+                    y = P.gelu_tanh(h @ d["feed_forward.w_up"].T) @ d["feed_forward.w_down"].T
+                want = P.stream_write(want, d["feed_forward_streams.mix"], d["feed_forward_streams.out"], y)
+            assert rel_err(X.permute(1, 0, 2), want) < tol, (ff, rows)
+
+
+# --------------------------------------------------------------------------- the convolution and the cell
+@pytest.mark.parametrize("K_", [1, 2, 3, 4, 6])
+@pytest.mark.parametrize("C,column,extra", [(32, 8, 4), (30, 5, 1), (1100, 4, 0)])
+def test_the_convolution_with_its_bias_from_a_column_on(K_, C, column, extra):
+    """Portions of unequal sizes (shorter than the taps among them), then single tokens, whose
+    kernel moves the tails itself; a result does not depend on which kernel made it."""
+    from gpt_fast_amd.ops import short_conv as SC
+    g = torch.Generator().manual_seed(C + K_)
+    lens, slots = [61, 9, 4], [3, 0, 2]
+    rows = [torch.randn(n, column + C + extra, generator=g, dtype=F) for n in lens]
+    taps, bias = torch.randn(C, K_, generator=g, dtype=F), torch.randn(C, generator=g, dtype=F)
+    for with_bias in (True, False):
+        state = torch.zeros(5, 8 + (K_ - 1) * C, dtype=torch.float32, device=DEV)
+        state[1].fill_(float("nan"))
+        got = [[] for _ in lens]
+        fed = [0, 0, 0]
+        for portion in ([40, 1, 2], [1, 1, 1], [17, 5, 0], [1, 1, 0], [1, 1, 1], [1, 0, 0]):
+            live = [b for b in range(3) if portion[b]]
+            take = [portion[b] for b in live]
+            x = _f32(torch.cat([rows[b][fed[b]:fed[b] + n] for b, n in zip(live, take)]))
+            q_start = _ints([sum(take[:i]) for i in range(len(take) + 1)])
+            tok_seq = _ints([i for i, n in enumerate(take) for _ in range(n)])
+            args = (x, _f32(taps), state, 8, tok_seq, q_start, _ints([slots[b] for b in live]), len(live))
+            kw = dict(bias=_f32(bias) if with_bias else None, column=column)
+            if max(take) == 1:
+                before = state.clone()
+                slow = SC.short_conv(*args, **kw)                  # the other kernel, on a copy of the tails
+                after = state.clone()
+                state.copy_(before)
+            y = SC.short_conv(*args, **kw, max_q_len=max(take))
+            if max(take) == 1:
+                assert torch.equal(y, slow) and torch.equal(state.nan_to_num(), after.nan_to_num())
+            at = 0
+            for b, n in zip(live, take):
+                got[b].append(y[at:at + n].double().cpu())
+                at += n
+                fed[b] += n
+        for b, n in enumerate(lens):
+            x = rows[b][:fed[b], column:column + C]
+            want = P.silu(P.short_convolution(x, taps, bias if with_bias else torch.zeros(C, dtype=F)))
+            assert rel_err(torch.cat(got[b]), want) < 1e-5
+            if K_ > 1 and fed[b] >= K_ - 1:
+                assert rel_err(state[slots[b], 8:].view(K_ - 1, C), x[-(K_ - 1):]) < 1e-6
+        assert torch.isnan(state[1]).all()
+
+
+@pytest.mark.parametrize("chunked", [0, 32, 64])
+@pytest.mark.parametrize("H,G,N,dv", [(6, 3, 24, 16), (1, 1, 12, 40), (4, 4, 6, 10), (8, 2, 128, 64), (2, 1, 136, 33),
+                                      (3, 1, 70, 144)])
+def test_the_cell_with_carried_state_token_by_token_and_in_chunks(H, G, N, dv, chunked):
+    """Three sequences in scattered slots, fed in portions of unequal sizes (down to one and two
+    tokens); the state travels from step to step."""
+    from gpt_fast_amd.ops import state_space as SS
+    g = torch.Generator().manual_seed(H * 31 + N)
+    layout = SS.RowLayout.fused(H, dv, G, N)
+    C, inner = layout.conv, H * dv
+    lens, slots = [150, 9, 70], [5, 0, 3]
+    conv = [torch.randn(n, C, generator=g, dtype=F) for n in lens]
+    proj = [torch.randn(n, layout.width, generator=g, dtype=F) * 2 for n in lens]
+    A_log, dt_bias = torch.rand(H, generator=g, dtype=F) * 5 - 4, torch.randn(H, generator=g, dtype=F) - 1
+    skip = torch.randn(H, generator=g, dtype=F)
+    state = torch.zeros(7, H * N * dv + 4, dtype=torch.float32, device=DEV)
+    state[1].fill_(float("nan"))                                     # a slot nobody owns
+    fed, got = [0, 0, 0], [[] for _ in lens]
+    for portion in ([1, 2, 70], [2, 1, 0], [100, 1, 0], [7, 5, 0], [40, 0, 0]):
+        live = [b for b in range(3) if portion[b]]
+        take = [portion[b] for b in live]
+        cut = lambda rows: _f32(torch.cat([rows[b][fed[b]:fed[b] + n] for b, n in zip(live, take)]))
+        q_start = _ints([sum(take[:i]) for i in range(len(take) + 1)])
+        y = SS.scan(cut(conv), cut(proj), layout, _f32(A_log), _f32(dt_bias), _f32(skip), state, q_start,
+                    _ints([slots[b] for b in live]), len(live), H, G, N, dv, chunked=bool(chunked), max_q_len=chunked)
+        at = 0
+        for b, n in zip(live, take):
+            got[b].append(y[at:at + n].double().cpu())
+            at += n
+            fed[b] += n
+    assert fed == lens
+    for b in range(3):
+        x, B, C_ = conv[b][:, :inner], conv[b][:, inner:inner + G * N], conv[b][:, inner + G * N:]
+        dt = P.softplus(proj[b][:, layout.dt:layout.dt + H] + dt_bias)
+        T = lens[b]
+        want = P.state_space(x.view(T, H, dv), B.view(T, G, N), C_.view(T, G, N), dt, A_log, skip)
+        assert rel_err(torch.cat(got[b]).view(T, H, dv), want) < 1e-4, b
+    assert torch.isnan(state[1]).all()
+
+
+def test_the_cell_forgets_at_once_and_not_at_all():
+    """A huge rate: the state is its last write, y_t = (dt B.C + D) x_t, nothing overflows.  A
+    rate near zero: the first token's write is read back 300 tokens later."""
+    from gpt_fast_amd.ops import state_space as SS
+    H, G, N, dv, T = 2, 1, 16, 16, 300
+    layout = SS.RowLayout.fused(H, dv, G, N)
+    conv = torch.zeros(T, layout.conv, dtype=F)
+    proj = torch.zeros(T, layout.width, dtype=F)
+    proj[:, layout.dt:layout.dt + H] = 3.0
+    g = torch.Generator().manual_seed(1)
+    for A_log, lasting in ((9.0, False), (-12.0, True)):
+        conv[:] = torch.randn(T, layout.conv, generator=g, dtype=F)
+        if lasting:
+            conv[1:, H * dv:H * dv + N] = 0.0                        # only the first token writes
+        for chunked in (0, 32, 64):
+            state = torch.zeros(1, H * N * dv, dtype=torch.float32, device=DEV)
+            y = SS.scan(_f32(conv), _f32(proj), layout, torch.full((H,), A_log, device=DEV),
+                        torch.zeros(H, device=DEV), torch.full((H,), 0.5, device=DEV), state, _ints([0, T]), _ints([0]),
+                        1, H, G, N, dv, chunked=bool(chunked), max_q_len=chunked)
+            dt = float(torch.nn.functional.softplus(torch.tensor(3.0, dtype=F)))
+            x = conv[:, :H * dv].view(T, H, dv)
+            B, C_ = conv[:, H * dv:H * dv + N], conv[:, H * dv + N:]
+            if lasting:
+                decay = torch.exp(-torch.exp(torch.tensor(A_log, dtype=F)) * dt * torch.arange(T, dtype=F))
+                want = (decay * dt * (C_ @ B[0]))[:, None, None] * x[0] + 0.5 * x
+            else:
+                want = (dt * (B * C_).sum(-1) + 0.5)[:, None, None] * x
+            assert rel_err(y.view(T, H, dv), want) < 1e-5, (A_log, chunked)
+
+
+@pytest.mark.parametrize("chunked", [32, 64])
+def test_a_fast_decay_does_not_cost_the_slow_ones_behind_it_their_digits(chunked):
+    """The logarithms of the decays sum up to -2,000 at one token of a chunk; the tokens behind
+    it decay by a hundredth each and are compared to seven digits."""
+    from gpt_fast_amd.ops import state_space as SS
+    H, G, N, dv, T = 1, 1, 16, 16, 30
+    layout = SS.RowLayout.fused(H, dv, G, N)
+    g = torch.Generator().manual_seed(3)
+    conv = torch.rand(T, layout.conv, generator=g, dtype=F) + 0.5
+    proj = torch.full((T, layout.width), -4.6, dtype=F)
+    proj[3] = 2000.0
+    conv[3] = 0.0
+    state = torch.zeros(1, H * N * dv, dtype=torch.float32, device=DEV)
+    y = SS.scan(_f32(conv), _f32(proj), layout, torch.zeros(H, device=DEV), torch.zeros(H, device=DEV),
+                torch.zeros(H, device=DEV), state, _ints([0, T]), _ints([0]), 1, H, G, N, dv, chunked=True,
+                max_q_len=chunked)
+    dt = P.softplus(proj[:, layout.dt:layout.dt + H])
+    want = P.state_space(conv[:, :dv].view(T, H, dv), conv[:, dv:dv + N].view(T, G, N), conv[:, dv + N:].view(T, G, N),
+                         dt, torch.zeros(H, dtype=F), torch.zeros(H, dtype=F))
+    assert rel_err(y.view(T, H, dv)[4:], want[4:]) < 2e-6
+
+
+@pytest.mark.parametrize("width,groups,offset", [(96, 4, 0), (96, 1, 8), (30, 3, 5), (2048, 8, 0), (6000, 2, 4), (40, 20, 4)])
+def test_the_gate_before_the_norm(width, groups, offset):
+    import dataclasses
+
+    from gpt_fast_amd.ops import decayed_memory as DM
+    g = torch.Generator().manual_seed(width + groups)
+    n = 7
+    y, z = torch.randn(n, width, generator=g, dtype=F), torch.randn(n, offset + width + 8, generator=g, dtype=F)
+    w = torch.rand(width, generator=g, dtype=F) + 0.5
+    layout = dataclasses.replace(DM.RowLayout.fused(1, 1, 1), width=offset + width + 8, g=offset)
+    want = P.gated_group_norm(y, z[:, offset:offset + width], w, groups, 1e-2)
+    for dtype, tol in ((torch.float32, 1e-5), (torch.bfloat16, 1e-2)):
+        got = DM.row_norm_gate(_f32(y), _f32(w), _f32(z), layout, 1e-2, dtype, groups=groups, gate="silu", gate_first=True)
+        assert rel_err(got, want) < tol
+    # it is another thing than the gate after the norm
+    after = DM.row_norm_gate(_f32(y), _f32(w), _f32(z), layout, 1e-2, torch.float32, groups=groups, gate="silu")
+    assert rel_err(after, want) > 1e-2
+
+
+# --------------------------------------------------------------------------- latents and their attention
+@pytest.mark.parametrize("dtype,tol", [(torch.float32, 1e-5), (torch.bfloat16, 1e-2)])
+@pytest.mark.parametrize("H,d,dr,R,Q,dims,scaling", [
+    (3, 16, 8, 32, 40, 8, (4.0, 64, 16.0, 2.0)), (2, 12, 8, 20, 28, 4, None), (4, 8, 16, 144, 24, 16, (2.0, 16, 1000.0, 500.0)),
+    (2, 10, 6, 10, 14, 2, None), (1, 8, 7, 16, 8, 6, None)])
+def test_latents_and_queries_with_half_split_rotation(dtype, tol, H, d, dr, R, Q, dims, scaling):
+    from gpt_fast_amd.config.spec import PositionSpec
+    from gpt_fast_amd.ops import scored_attention as SA
+    from gpt_fast_amd.parts.position import frequencies_and_trig_scale
+    g = torch.Generator().manual_seed(R + Q)
+    lens, starts = [70, 1, 3], [0, 130, 62]
+    n_pages, tables, table, tok_seq, tok_pos, pos = _table_and_positions(lens, starts)
+    N = sum(lens)
+    rot = {"dims": dims, "base": 77.0}
+    sc = None
+    if scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+        sc = (("rope_type", "yarn"),) + tuple(rot["scaling"].items())
+    freqs, trig = frequencies_and_trig_scale(PositionSpec(rotary_dim=dims, base=77.0, layout="half", scaling=sc))
+    freqs = freqs.to(DEV)
+    proj = torch.randn(N, Q + R + dr + 5, generator=g, dtype=F) * 2
+    wq, wkv = torch.rand(Q, generator=g, dtype=F) + 0.5, torch.rand(R, generator=g, dtype=F) + 0.5
+    k_pages = torch.zeros(n_pages, 1, 64, R + dr, device=DEV, dtype=dtype)
+    v_pages = torch.zeros(n_pages, 1, R, 64, device=DEV, dtype=dtype)
+    cq = SA.latent_store(_f32(proj), Q, R, dr, _f32(wq), _f32(wkv), 1e-4, freqs, dims, tok_seq, tok_pos, table,
+                         k_pages, v_pages, dtype, layout=1, trig_scale=trig)
+    positions = torch.tensor(pos)
+    assert rel_err(cq, P.rms_norm(proj[:, :Q], wq, 1e-4)) < tol
+    want_c = P.rms_norm(proj[:, Q:Q + R], wkv, 1e-4)
+    want_kr = P.rotate_half(proj[:, None, Q + R:Q + R + dr], positions, rot)[:, 0]
+    k = k_pages.reshape(n_pages, 1, -1)[..., util.key_places(R + dr).reshape(-1)].view(n_pages, 64, R + dr)
+    v = v_pages.reshape(n_pages, 1, -1)[..., util.value_places(R).reshape(-1)].view(n_pages, R, 64)
+    seqs = [b for b, l in enumerate(lens) for _ in range(l)]
+    for n, (b, p_) in enumerate(zip(seqs, pos)):
+        page = tables[b][p_ // 64]
+        assert rel_err(k[page, p_ % 64, :R], want_c[n]) < tol
+        assert rel_err(k[page, p_ % 64, R:], want_kr[n]) < tol
+        assert rel_err(v[page, :, p_ % 64], want_c[n]) < tol
+    q = torch.randn(N, H * (d + dr), generator=g, dtype=F)
+    plain, full = SA.latent_query(_f32(q), freqs, dims, tok_pos, H, d, dr, R, dtype, layout=1, trig_scale=trig)
+    qq = q.view(N, H, d + dr)
+    assert rel_err(plain.permute(1, 0, 2), qq[..., :d]) < tol
+    assert rel_err(full.permute(1, 0, 2)[..., R:], P.rotate_half(qq[..., d:], positions, rot)) < tol
+
+
+@pytest.mark.parametrize("dtype,tol", [(torch.float32, 2e-5), (torch.bfloat16, 2e-2)])
+@pytest.mark.parametrize("H,hd,vd", [(6, 64, 48), (3, 24, 20), (1, 96, 64), (12, 160, 144), (2, 576, 512)])
+def test_the_attention_gates_its_heads_and_finds_a_key_that_stands_out(dtype, tol, H, hd, vd):
+    """One kv head for all; a loud key at page borders and at the start takes all the weight; the
+    pool beyond the sequences' ends is not a number.  Prompts, portions and single tokens, with
+    the kernel that works token by token and with the matrix-core kernel."""
+    from gpt_fast_amd.ops import scored_attention as SA
+    for lens, starts, loud in (([130, 3], [0, 0], None), ([37, 2, 1], [100, 63, 64], (0, 0)), ([1, 1, 1], [63, 64, 300], (2, 63)),
+                               ([1, 1], [200, 127], (0, 128)), ([70], [64], (0, 64))):
+        g = torch.Generator().manual_seed(H + hd)
+        total = [s + l for s, l in zip(starts, lens)]
+        n_pages, tables, table, _, _, _ = _table_and_positions(total, [0] * len(total))
+        ks = [torch.randn(t, hd, generator=g, dtype=F) for t in total]
+        vs = [torch.randn(t, vd, generator=g, dtype=F) for t in total]
+        qs = [torch.randn(l, H, hd, generator=g, dtype=F) for l in lens]
+        if loud is not None:
+            b, j = loud
+            qs[b][:, :, 0] = 3.0
+            ks[b][:, 0] = 0.0
+            ks[b][j, 0] = 60.0
+        if dtype == torch.bfloat16:
+            ks, vs, qs = ([t.to(dtype).double() for t in ts] for ts in (ks, vs, qs))
+        k_pages = torch.full((n_pages + 1, 1, 64, hd), float("nan"), dtype=dtype, device=DEV)
+        v_pages = torch.full((n_pages + 1, 1, vd, 64), float("nan"), dtype=dtype, device=DEV)
+        rows = torch.cat([torch.cat([torch.zeros(t, hd, dtype=F), k, v], 1) for t, k, v in zip(total, ks, vs)])
+        SA.unit_heads_store(_f32(rows), None, _ints([b for b, t in enumerate(total) for _ in range(t)]),
+                            _ints([i for t in total for i in range(t)]), table, k_pages, v_pages, 1, 1, hd, vd, None, dtype)
+        tok_seq = _ints([b for b, l in enumerate(lens) for _ in range(l)])
+        tok_pos = _ints([s + i for s, l in zip(starts, lens) for i in range(l)])
+        q_start = _ints([sum(lens[:b]) for b in range(len(lens) + 1)])
+        gate = torch.randn(sum(lens), H + 3, generator=g, dtype=F) * 2
+        want = torch.zeros(sum(lens), H, vd, dtype=F)
+        at = 0
+        for b, l in enumerate(lens):
+            for i in range(l):
+                p = torch.softmax(qs[b][i] @ ks[b][:starts[b] + i + 1].T * 0.25, -1)
+                want[at] = (p @ vs[b][:starts[b] + i + 1]) * torch.sigmoid(gate[at, 2:2 + H])[:, None]
+                at += 1
+        q = torch.cat(qs).to(dtype).to(DEV)
+        for head_major in (False, True):
+            qq = q.permute(1, 0, 2).contiguous() if head_major else q
+            for step in (None, (q_start, _ints(starts), len(lens), max(lens))):
+                got = SA.attention(qq, k_pages, v_pages, tok_seq, tok_pos, table, 0.25, head_major=head_major,
+                                   gate=_f32(gate)[:, 2:], step=step)
+                assert rel_err(got.permute(1, 0, 2) if head_major else got, want) < tol, (lens, starts, head_major)
+
+
+# --------------------------------------------------------------------------- whole models
+@pytest.mark.parametrize("name", sorted(CASES))
+@pytest.mark.parametrize("dtype,tol", [("float32", TOL_F32_LONG), ("bfloat16", TOL_BF16)])
+def test_whole_prompt_at_every_position_and_the_streams_sum_after_every_run(tmp_path, name, dtype, tol):
+    folder = make_folder(tmp_path, name, seed=11)
+    cfg, w = P.load_folder(folder)
+    toks = util.random_tokens(cfg["vocab"], 150, 3)
+    outs = []
+    want = P.forward(w, cfg, toks, outs)
+    eng = _engine(folder, dtype)
+    taps = []
+    eng.model.tap = lambda n, x: taps.append(x.double().cpu())
+    got = _steps(eng, toks, [])
+    eng.model.tap = None
+    assert close(got, want, dtype, tol)
+    assert len(taps) == len(outs) == len(P.run_order(cfg))
+    if dtype == "float32":
+        for n, (a, b) in enumerate(zip(taps, outs)):
+            assert rel_err(a, b) < TOL_F32_LONG, n
+        # one token, and the first tokens of a sequence (fewer than the taps)
+        assert rel_err(_steps(eng, toks[:1], []), want[:1]) < TOL_F32_LONG
+        assert rel_err(_steps(eng, toks[:3], []), want[:3]) < TOL_F32_LONG
+        assert rel_err(_steps(eng, toks[:3], [1, 2]), want[:3]) < TOL_F32_LONG
+
+
+@pytest.mark.parametrize("name", sorted(CASES))
+@pytest.mark.parametrize("dtype,tol", [("float32", TOL_F32_LONG), ("bfloat16", TOL_BF16)])
+def test_portions_and_token_by_token_equal_the_whole_prompt(tmp_path, name, dtype, tol):
+    folder = make_folder(tmp_path, name, seed=12)
+    cfg, w = P.load_folder(folder)
+    toks = util.random_tokens(cfg["vocab"], 210, 5)
+    want = P.forward(w, cfg, toks)
+    eng = _engine(folder, dtype)
+    whole = _steps(eng, toks, [])
+    assert close(whole, want, dtype, tol)
+    for cuts in ([2, 4, 5, 70, 128, 129], [63, 64, 65, 192], [17, 150], list(range(150, 210)),
+                 list(range(1, 80)), list(range(2, 210, 2))):
+        got = _steps(eng, toks, cuts)
+        assert close(got, want, dtype, tol), cuts
+        assert close(got, whole, dtype, tol), cuts
+    eng.cache.check()
+
+
+@pytest.mark.parametrize("name", ["A", "B", "C"])
+@pytest.mark.parametrize("dtype,same", [("float32", 2e-5), ("bfloat16", TOL_BF16)])
+def test_unequal_batches_equal_each_request_alone(tmp_path, name, dtype, same):
+    import gpt_fast_amd as gfa
+    folder = make_folder(tmp_path, name, seed=13)
+    cfg, w = P.load_folder(folder)
+    lens = [1, 5, 131, 64, 70]
+    tail = 30
+    seqs = [util.random_tokens(cfg["vocab"], n + tail, 40 + n) for n in lens]
+    eng = _engine(folder, dtype, max_tokens=64 * 20, max_sequences=6)
+    alone = [_steps(eng, s, [n] + list(range(n + 1, n + tail))) for s, n in zip(seqs, lens)]
+    slots = [eng.start_sequence() for _ in seqs]
+    got = [[] for _ in seqs]
+    out = eng.step([gfa.Entry(sl, s[:n], want=list(range(n))) for sl, s, n in zip(slots, seqs, lens)]).cpu()
+    at = 0
+    for b, n in enumerate(lens):
+        got[b].append(out[at:at + n])
+        at += n
+    live = list(range(len(seqs)))
+    for t in range(tail):
+        if t == 10:                                  # a shorter request ends earlier
+            eng.end_sequence(slots[1])
+            live.remove(1)
+        out = eng.step([gfa.Entry(slots[b], [seqs[b][lens[b] + t]], want=[0]) for b in live]).cpu()
+        for i, b in enumerate(live):
+            got[b].append(out[i:i + 1])
+    for b in live:
+        eng.end_sequence(slots[b])
+    eng.cache.check()
+    for b, s in enumerate(seqs):
+        g = torch.cat(got[b])
+        assert close(g, alone[b][:g.shape[0]], dtype, same), b
+    want = P.forward(w, cfg, seqs[2])
+    assert close(torch.cat(got[2]), want, dtype, TOL_F32_LONG)
+
+
+@pytest.mark.parametrize("name", ["A", "C"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_a_step_that_mixes_single_tokens_a_portion_and_a_new_prompt(tmp_path, name, dtype):
+    import gpt_fast_amd as gfa
+    folder = make_folder(tmp_path, name, seed=21)
+    cfg, w = P.load_folder(folder)
+    _, before, mixed = util.mixed_step_case(cfg["vocab"])
+    lens = {"d0": 9, "d1": 66, "d2": 130, "c": 112, "p": 131}
+    seqs = {r: util.random_tokens(cfg["vocab"], n, 300 + n) for r, n in lens.items()}
+    eng = _engine(folder, dtype, max_tokens=64 * 16, max_sequences=5)
+    slots = {r: eng.start_sequence() for r in seqs}
+    got = {r: [] for r in seqs}
+    fed = {r: 0 for r in seqs}
+
+    def step(order, portions):
+        logits = eng.step([gfa.Entry(slots[r], seqs[r][fed[r]:fed[r] + portions[r]], want=list(range(portions[r])))
+                           for r in order]).cpu()
+        at = 0
+        for r in order:
+            got[r].append(logits[at:at + portions[r]])
+            at += portions[r]
+            fed[r] += portions[r]
+    step(["d0", "d1", "d2", "c"], before)
+    step(["d0", "c", "d1", "p", "d2"], mixed)
+    for r in ("c", "p"):
+        while fed[r] < len(seqs[r]):
+            step([r], {r: 1})
+    for r in seqs:
+        eng.end_sequence(slots[r])
+    eng.cache.check()
+    assert eng.cache.slots.held == 0
+    for r, toks in seqs.items():
+        assert close(torch.cat(got[r]), P.forward(w, cfg, toks)[:fed[r]], dtype, TOL_F32_LONG), r
+
+
+@pytest.mark.parametrize("batch", [12, 20, 40])
+def test_wide_decoding_steps_take_the_larger_products_kernels(tmp_path, batch):
+    """A dozen to forty requests decode together: the products' kernels change with the number
+    of rows, the results do not."""
+    import gpt_fast_amd as gfa
+    folder = make_folder(tmp_path, "C", seed=27)
+    cfg, w = P.load_folder(folder)
+    seqs = [util.random_tokens(cfg["vocab"], 3 + b % 5 + 6, 500 + b) for b in range(batch)]
+    eng = _engine(folder, "bfloat16", max_tokens=64 * batch, max_sequences=batch)
+    slots = [eng.start_sequence() for _ in seqs]
+    got = [[] for _ in seqs]
+    eng.step([gfa.Entry(sl, s[:-6], want=[]) for sl, s in zip(slots, seqs)])
+    for t in range(6):
+        out = eng.step([gfa.Entry(sl, [s[len(s) - 6 + t]], want=[0]) for sl, s in zip(slots, seqs)]).cpu()
+        for b in range(batch):
+            got[b].append(out[b:b + 1])
+    for b, s in enumerate(seqs):
+        assert close(torch.cat(got[b]), P.forward(w, cfg, s)[-6:], "bfloat16", None), b
+
+
+def test_slots_and_pages_that_come_back_start_clean(tmp_path):
+    """A cache of few pages and two slots: requests follow one another in the same slots and
+    pages (the cell's state and the convolution's tails of every run among their state), and
+    every request equals the plain computation of itself alone."""
+    import gpt_fast_amd as gfa
+    folder = make_folder(tmp_path, "A", seed=14)
+    cfg, w = P.load_folder(folder)
+    eng = _engine(folder, "float32", max_tokens=64 * 7, max_sequences=2)
+    for again in range(3):
+        a = util.random_tokens(cfg["vocab"], 150 + 60, 60 + again)
+        b = util.random_tokens(cfg["vocab"], 40 + 60, 70 + again)
+        sa, sb = eng.start_sequence(), eng.start_sequence()
+        assert {sa, sb} == {0, 1}
+        got_a, got_b = [], []
+        out = eng.step([gfa.Entry(sa, a[:150], want=[149]), gfa.Entry(sb, b[:40], want=[39])]).cpu()
+        got_a.append(out[0:1])
+        got_b.append(out[1:2])
+        for t in range(59):
+            out = eng.step([gfa.Entry(sa, [a[150 + t]], want=[0]), gfa.Entry(sb, [b[40 + t]], want=[0])]).cpu()
+            got_a.append(out[0:1])
+            got_b.append(out[1:2])
+        eng.cache.check()
+        eng.end_sequence(sb)
+        eng.end_sequence(sa)
+        assert rel_err(torch.cat(got_a), P.forward(w, cfg, a[:-1])[149:]) < TOL_F32_LONG
+        assert rel_err(torch.cat(got_b), P.forward(w, cfg, b[:-1])[39:]) < TOL_F32_LONG
+    for _, g in eng.cache.paged_groups:
+        assert g.pages.held == 0
+
+
+@pytest.mark.parametrize("far", [0, 63, 64, 127, 128])
+def test_a_far_key_in_a_whole_model_in_prompts_and_in_decoding(tmp_path, far):
+    """One attention layer whose scores are large, so that single keys decide: one token far back,
+    at a page's border, is replaced, and the logits of the positions that look for it change as
+    the plain implementation says; whole, in portions and decoded."""
+    config = dict(CASES["A"])
+    config["layers"] = [config["layers"][0]]
+    config["loop"] = {"start": 0, "stop": 1, "times": 2}
+
+    def patch(t):
+        t["l0.mix.uq"] = t["l0.mix.uq"] * 12
+    folder = write_model(os.path.join(str(tmp_path), f"far{far}"), config, 40, patch=patch)
+    cfg, w = P.load_folder(folder)
+    T = 260
+    toks = util.random_tokens(cfg["vocab"], T, 5)
+    other = list(toks)
+    other[far] = (other[far] + 7) % cfg["vocab"]
+    wants = [P.forward(w, cfg, s) for s in (toks, other)]
+    changed = row_errors(wants[1], wants[0])[far + 100:]
+    assert float(changed.max()) > 0.03                                # the far key matters
+    eng = _engine(folder, "float32", max_tokens=64 * 8, max_sequences=1)
+    for s, want in zip((toks, other), wants):
+        for cuts in ([], [far + 1, far + 3] if far else [2], [200] + list(range(201, T))):
+            assert rel_err(_steps(eng, s, cuts), want) < 5 * TOL_F32_LONG, cuts
+    eng = _engine(folder, "bfloat16", max_tokens=64 * 8, max_sequences=1)
+    for s, want in zip((toks, other), wants):
+        got = _steps(eng, s, [200] + list(range(201, T)))
+        assert float(row_errors(got, want).median()) < 2 * TOL_BF16
+    eng.cache.check()
+
+
+def test_state_that_lasts_hundreds_of_tokens_and_long_decoding(tmp_path):
+    """Decays next to one: the first tokens decide the last logits five hundred tokens later,
+    through a prompt and 130 tokens decoded one by one."""
+    config = dict(CASES["A"])
+    config["layers"] = [config["layers"][1], config["layers"][3]]
+    config["loop"] = {"start": 1, "stop": 2, "times": 2}
+
+    def patch(t):
+        for name in t:
+            if name.endswith(".A_log"):
+                t[name] = torch.full_like(t[name], -8.0)
+    folder = write_model(os.path.join(str(tmp_path), "lasting"), config, 16, patch=patch)
+    cfg, w = P.load_folder(folder)
+    toks = util.random_tokens(cfg["vocab"], 520, 21)
+    want = P.forward(w, cfg, toks)
+    # it matters: with other first tokens the last logits are others
+    other = util.random_tokens(cfg["vocab"], 20, 22) + toks[20:]
+    assert rel_err(P.forward(w, cfg, other)[-40:], want[-40:]) > 1e-2
+    for dtype in ("float32", "bfloat16"):
+        eng = _engine(folder, dtype, max_tokens=64 * 10, max_sequences=1)
+        got = _steps(eng, toks, [390] + list(range(391, 520)))
+        assert close(got, want, dtype, 3 * TOL_F32_LONG)
+        eng.cache.check()
+
+
+@pytest.mark.parametrize("seed", [1, 2, 3, 4, 5, 6, 7, 8])
+def test_random_configurations_whole_and_in_a_batch_that_is_decoded_together(tmp_path, seed):
+    """Sizes drawn at random (bikadra_cases.random_case): requests of 300, 130, 33 and 1 tokens,
+    each whole, then their prompts in one batch and twenty tokens decoded together."""
+    import gpt_fast_amd as gfa
+    config = random_case(seed)
+    folder = write_model(os.path.join(str(tmp_path), f"random{seed}"), config, 100 + seed, std=0.05)
+    cfg, w = P.load_folder(folder)
+    lens = [300, 130, 33, 1]
+    seqs = [util.random_tokens(cfg["vocab"], n + 20, 7 * seed + n) for n in lens]
+    want = [P.forward(w, cfg, s) for s in seqs]
+    for dtype in ("float32", "bfloat16"):
+        eng = _engine(folder, dtype, max_tokens=4096, max_sequences=4)
+        for s, wanted in zip(seqs, want):
+            assert close(_steps(eng, s, []), wanted, dtype, 3 * TOL_F32_LONG), (dtype, len(s))
+        slots = [eng.start_sequence() for _ in seqs]
+        got = [[] for _ in seqs]
+        out = eng.step([gfa.Entry(sl, s[:n], want=list(range(n))) for sl, s, n in zip(slots, seqs, lens)]).cpu()
+        at = 0
+        for b, n in enumerate(lens):
+            got[b].append(out[at:at + n])
+            at += n
+        for t in range(20):
+            out = eng.step([gfa.Entry(slots[b], [seqs[b][lens[b] + t]], want=[0]) for b in range(len(seqs))]).cpu()
+            for b in range(len(seqs)):
+                got[b].append(out[b:b + 1])
+        for sl in slots:
+            eng.end_sequence(sl)
+        eng.cache.check()
+        for b in range(len(seqs)):
+            assert close(torch.cat(got[b]), want[b], dtype, 3 * TOL_F32_LONG), (dtype, b)
+
+
+# --------------------------------------------------------------------------- generation
+@pytest.mark.parametrize("name", ["A", "C"])
+def test_greedy_generation_through_the_loop_and_the_recorded_step(tmp_path, name):
+    from gpt_fast_amd.engine.generate import generate
+    folder = make_folder(tmp_path, name, seed=17)
+    cfg, w = P.load_folder(folder)
+    prompts = [util.random_tokens(cfg["vocab"], n, 80 + n) for n in (7, 1, 90, 30)]
+    want = [P.greedy_generate(w, cfg, p, 12) for p in prompts]
+    eng = _engine(folder, "float32", max_tokens=64 * 12, max_sequences=4)
+    assert eng.model.replayable
+    for use_graph in (False, True, True):                       # the recording is replayed
+        got = generate(eng, prompts, max_new_tokens=12, temperature=0.0, use_graph=use_graph)
+        assert got.tokens == want, use_graph
+    # two at a time: slots and state come back between the batches
+    got = generate(eng, prompts, max_new_tokens=12, temperature=0.0, batch_size=2)
+    assert got.tokens == want
+    eng.cache.check()
+    # bfloat16 through the recorded step: the tokens of the step that is not recorded
+    eng = _engine(folder, "bfloat16", max_tokens=64 * 12, max_sequences=4)
+    plain_steps = generate(eng, prompts, max_new_tokens=12, temperature=0.0, use_graph=False).tokens
+    for _ in range(2):
+        assert generate(eng, prompts, max_new_tokens=12, temperature=0.0, use_graph=True).tokens == plain_steps
+
+
+def test_command_line_entry_point(tmp_path):
+    import gpt_fast_amd as gfa
+    folder = make_folder(tmp_path, "B", seed=18)
+    cfg, w = P.load_folder(folder)
+    prompt = util.random_tokens(cfg["vocab"], 20, 1)
+    lines = []
+    res = gfa.main(prompt=prompt, num_samples=1, max_new_tokens=8, temperature=0.0, top_k=None,
+                   checkpoint_path=folder, dtype="float32", device=DEV, out=lines.append)
+    assert res["result"].tokens[0] == P.greedy_generate(w, cfg, prompt, 8)
+    assert any("tokens/sec" in str(l) for l in lines)
+
+
+def test_trace_replay_program(tmp_path):
+    """bin/trace_run as a program on a Bikadra folder: two batches of unequal requests one after
+    the other (the second takes the slots, state and pages the first gave back), logits wanted
+    at some places only, steps in which nothing is wanted, a request that ends in the step that
+    brings its prompt."""
+    import json
+    import subprocess
+
+    import numpy as np
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    folder = make_folder(tmp_path, "A", seed=19)
+    cfg, w = P.load_folder(folder)
+    V = cfg["vocab"]
+    reqs = {"a": util.random_tokens(V, 140, 1), "b": util.random_tokens(V, 9, 2), "c": util.random_tokens(V, 1, 3),
+            "d": util.random_tokens(V, 150, 4), "e": util.random_tokens(V, 70, 5)}
+    prompt = {"a": 120, "b": 3, "c": 1, "d": 130, "e": 64}
+    steps, where = [], {r: [] for r in reqs}          # request -> (step, row in the file, position)
+    n = 0
+    for ids in (["a", "b", "c"], ["d", "e"]):
+        live, t = list(ids), 0
+        while live:
+            entries, row = [], 0
+            for r in live:
+                lo, hi = (0, prompt[r]) if t == 0 else (prompt[r] + t - 1, prompt[r] + t)
+                want = [i for i in range(hi - lo) if (lo + i) % 3 != 1]
+                entries.append({"id": r, "tokens": reqs[r][lo:hi], "want": want})
+                for i in want:
+                    where[r].append((n, row, lo + i))
+                    row += 1
+            ends = [r for r in live if (prompt[r] + t if t else prompt[r]) >= len(reqs[r])]
+            steps.append({"step": n, "entries": entries, "end": ends})
+            live = [r for r in live if r not in ends]
+            n += 1
+            t += 1
+    for dtype in ("float32", "bfloat16"):
+        out_dir = os.path.join(str(tmp_path), "out_" + dtype)
+        proc = subprocess.run(
+            [os.path.join(root, "bin", "trace_run"), "--model", folder, "--dtype", dtype, "--out", out_dir,
+             "--max-tokens", "400"],
+            input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=600)
+        assert proc.returncode == 0, proc.stderr[-2000:]
+        assert [l for l in proc.stdout.splitlines() if l.startswith("done ")] == [f"done {i}" for i in range(n)]
+        for r, toks in reqs.items():
+            if not where[r]:
+                continue
+            got = torch.stack([torch.from_numpy(np.fromfile(os.path.join(out_dir, f"{s}.f32"), dtype="<f4")
+                                                .reshape(-1, V)[row]) for s, row, _ in where[r]])
+            want = P.forward(w, cfg, toks)[[p for _, _, p in where[r]]]
+            assert close(got, want, dtype, TOL_F32_LONG), (dtype, r)
