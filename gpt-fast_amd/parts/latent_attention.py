@@ -4,6 +4,7 @@ import torch
 from ..cache.store import KVNeed
 from ..config.spec import LatentAttentionSpec
 from ..ops import kernels as K
+from ..ops import latent_attention as LA
 from ..ops import linear as L
 from ..ops import scored_attention as SA
 from .base import Param, Part, Runtime, add_late, check_bound, register_mixer
@@ -35,7 +36,10 @@ class LatentAttention(Part):
     Without a query latent (``q_rank`` None) ``q = w_q x``: the kv down projection and ``w_q``
     are then one matrix over x, whose float32 sums serve both."""
 
-    libraries = ("scored_attention",)
+    @staticmethod
+    def libraries(runtime):
+        return ("scored_attention",) if runtime.is_float32 else ("scored_attention", "latent_attention")
+
     replayable = True
     defers_sum = True              # ``residual`` may be a parts.base.ResidualStream
 
@@ -129,10 +133,10 @@ class LatentAttention(Part):
                                       s.head_dim, s.rot_dim, R, self.rt.dtype, layout=self.layout,
                                       trig_scale=self.trig)
         self._per_head(plain, self.w_uk, full[:, :, :R])
-        latent = SA.attention(full, entry.k_pages, entry.v_pages, batch.tok_seq, batch.tok_pos,
-                              table, s.scale, window=self.window, head_major=True,
-                              gate=down[:, self.gate_at:self.down_rows] if s.head_gate else None,
-                              step=(batch.q_start, batch.start_pos, batch.n_seqs, batch.max_q_len))
+        latent = LA.attention(full, entry.k_pages, entry.v_pages, batch.tok_seq, batch.tok_pos, table,
+                              s.scale, (batch.q_start, batch.start_pos, batch.n_seqs, batch.max_q_len),
+                              window=self.window,
+                              gate=down[:, self.gate_at:self.down_rows] if s.head_gate else None)
         y = torch.empty((n, s.n_heads, s.value_dim), dtype=self.rt.dtype, device=x.device)
         self._per_head(latent, self.w_uv, y.permute(1, 0, 2))
         return y.view(n, s.n_heads * s.value_dim)

@@ -395,11 +395,13 @@ def test_latents_and_queries_with_half_split_rotation(dtype, tol, H, d, dr, R, Q
 
 
 @pytest.mark.parametrize("dtype,tol", [(torch.float32, 2e-5), (torch.bfloat16, 2e-2)])
-@pytest.mark.parametrize("H,hd,vd", [(6, 64, 48), (3, 24, 20), (1, 96, 64), (12, 160, 144), (2, 576, 512)])
+@pytest.mark.parametrize("H,hd,vd", [(6, 64, 48), (3, 24, 20), (1, 96, 64), (12, 160, 144), (2, 576, 512),
+                                     (20, 200, 144), (40, 72, 64), (70, 328, 272), (32, 576, 512)])
 def test_the_attention_gates_its_heads_and_finds_a_key_that_stands_out(dtype, tol, H, hd, vd):
     """One kv head for all; a loud key at page borders and at the start takes all the weight; the
     pool beyond the sequences' ends is not a number.  Prompts, portions and single tokens, with
-    the kernel that works token by token and with the matrix-core kernel."""
+    the kernel that works token by token and with the matrix-core kernels."""
+    from gpt_fast_amd.ops import latent_attention as LA
     from gpt_fast_amd.ops import scored_attention as SA
     for lens, starts, loud in (([130, 3], [0, 0], None), ([37, 2, 1], [100, 63, 64], (0, 0)), ([1, 1, 1], [63, 64, 300], (2, 63)),
                                ([1, 1], [200, 127], (0, 128)), ([70], [64], (0, 64))):
@@ -439,6 +441,59 @@ def test_the_attention_gates_its_heads_and_finds_a_key_that_stands_out(dtype, to
                 got = SA.attention(qq, k_pages, v_pages, tok_seq, tok_pos, table, 0.25, head_major=head_major,
                                    gate=_f32(gate)[:, 2:], step=step)
                 assert rel_err(got.permute(1, 0, 2) if head_major else got, want) < tol, (lens, starts, head_major)
+        # the kernels for one shared kv head: whole, and a single-token step's keys in parts
+        qq = q.permute(1, 0, 2).contiguous()
+        for n_parts in (None, 1, 2, 3, 64) if max(lens) == 1 else (None,):
+            got = LA.attention(qq, k_pages, v_pages, tok_seq, tok_pos, table, 0.25,
+                               (q_start, _ints(starts), len(lens), max(lens)), gate=_f32(gate)[:, 2:], n_parts=n_parts)
+            assert rel_err(got.permute(1, 0, 2), want) < tol, (lens, starts, n_parts)
+
+
+@pytest.mark.parametrize("window", [1, 31, 32, 33, 64, 100])
+@pytest.mark.parametrize("H,hd,vd", [(5, 72, 64), (32, 576, 512)])
+def test_one_shared_kv_head_with_a_window(H, hd, vd, window):
+    """The first key that is seen, and the one before it, are loud in turn; prompts, portions
+    and single tokens with the keys in one and in several parts; pages before the window hold no
+    number, as do those behind the end."""
+    from gpt_fast_amd.ops import latent_attention as LA
+    from gpt_fast_amd.ops import scored_attention as SA
+    for lens, starts in (([150], [0]), ([9], [120]), ([1, 1, 1], [40, 127, 200])):
+        for off in (0, -1):                                # just inside, just outside the last row's window
+            g = torch.Generator().manual_seed(window + H)
+            total = [s + l for s, l in zip(starts, lens)]
+            n_pages, tables, table, _, _, _ = _table_and_positions(total, [0] * len(total))
+            ks = [torch.randn(t, hd, generator=g, dtype=F) for t in total]
+            vs = [torch.randn(t, vd, generator=g, dtype=F) for t in total]
+            qs = [torch.randn(l, H, hd, generator=g, dtype=F) for l in lens]
+            for b, t in enumerate(total):
+                j = t - window + off
+                qs[b][:, :, 0] = 3.0
+                ks[b][:, 0] = 0.0
+                if 0 <= j < t:
+                    ks[b][j, 0] = 40.0
+            ks, vs, qs = ([t.bfloat16().double() for t in ts] for ts in (ks, vs, qs))
+            k_pages = torch.full((n_pages + 1, 1, 64, hd), float("nan"), dtype=torch.bfloat16, device=DEV)
+            v_pages = torch.full((n_pages + 1, 1, vd, 64), float("nan"), dtype=torch.bfloat16, device=DEV)
+            rows = torch.cat([torch.cat([torch.zeros(t, hd, dtype=F), k, v], 1) for t, k, v in zip(total, ks, vs)])
+            SA.unit_heads_store(_f32(rows), None, _ints([b for b, t in enumerate(total) for _ in range(t)]),
+                                _ints([i for t in total for i in range(t)]), table, k_pages, v_pages, 1, 1, hd, vd, None,
+                                torch.bfloat16)
+            for b, s in enumerate(starts):                 # pages nobody can see any more
+                for pg in range(max(0, s - window + 1) // 64):
+                    k_pages[tables[b][pg]] = float("nan")
+                    v_pages[tables[b][pg]] = float("nan")
+            want = []
+            for b, l in enumerate(lens):
+                for i in range(l):
+                    p = starts[b] + i
+                    lo = max(0, p - window + 1)
+                    want.append(torch.softmax(qs[b][i] @ ks[b][lo:p + 1].T * 0.25, -1) @ vs[b][lo:p + 1])
+            want = torch.stack(want)
+            q = torch.cat(qs).bfloat16().to(DEV).permute(1, 0, 2).contiguous()
+            step = (_ints([sum(lens[:b]) for b in range(len(lens) + 1)]), _ints(starts), len(lens), max(lens))
+            for n_parts in (None, 1, 2, 5) if max(lens) == 1 else (None,):
+                got = LA.attention(q, k_pages, v_pages, None, None, table, 0.25, step, window=window, n_parts=n_parts)
+                assert rel_err(got.permute(1, 0, 2), want) < 2e-2, (lens, starts, off, n_parts)
 
 
 # --------------------------------------------------------------------------- whole models
