@@ -82,6 +82,15 @@ __device__ __forceinline__ float block_max(float v, float* scratch) {
     return t;
 }
 
+// A workgroup barrier for data that is exchanged through shared memory only: it waits for this
+// wave's shared-memory accesses and for no global load or store, so that loads asked for ahead
+// stay in flight across it (__syncthreads waits for all of them).
+__device__ __forceinline__ void lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
+
 // Layout of the cache.  One layer's pool of keys, and its pool of values, gives every
 // (page, kv head) a region of GFA_PAGE * head_dim elements.  Inside a region the elements lie
 // in the order in which the matrix-core attention reads its operands, so that a wave's load

@@ -160,8 +160,9 @@ __device__ __forceinline__ sc_floatx4_t sc_mfma4(float4 a, float4 b, sc_floatx4_
     return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
 }
 
-// NV: 16-byte loads of B and of C per thread (0: plain loads)
-template <int SC_L, int NV>
+// NV: 16-byte loads of B and of C per thread (0: plain loads); NC: the number of states where it
+// is known (a multiple of 16: the products' loops are then unrolled), else 0
+template <int SC_L, int NV, int NC>
 __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
         const float* __restrict__ conv, const float* __restrict__ proj,
         const float* __restrict__ A_log, const float* __restrict__ dt_bias,
@@ -170,7 +171,8 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
         SSShape s, int n_cols, int n_seqs) {
     extern __shared__ __attribute__((aligned(16))) float sc_lds[];
     constexpr int NT = SC_L * 8, NW = NT / 64, TS = SC_L + 4;
-    const int KS = sc_row_stride(s.N), Np = sc_padded(s.N);
+    const int N = NC ? NC : s.N;
+    const int KS = sc_row_stride(N), Np = sc_padded(N);
     float* Cs = sc_lds;                          // [SC_L][KS]
     float* Bs = Cs + SC_L * KS;                  // [SC_L][KS]
     float* St = Bs + SC_L * KS;                  // [SC_COLS][KS]  S transposed
@@ -190,20 +192,20 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
     const int grp = h / (s.H / s.G), inner = s.H * s.dv;
     const int t0 = q_start[b], t1 = q_start[b + 1];
     if (t0 >= t1) return;                        // the whole workgroup
-    float* const S = state + (size_t)slots[b] * slot_stride + (size_t)h * s.N * s.dv;
+    float* const S = state + (size_t)slots[b] * slot_stride + (size_t)h * N * s.dv;
     const float rate = expf(A_log[h]), bias = dt_bias[h], Dh = skip[h];
-    const int b_col = inner + grp * s.N, c_col = inner + s.G * s.N + grp * s.N, x_col = h * s.dv + col0;
+    const int b_col = inner + grp * N, c_col = inner + s.G * N + grp * N, x_col = h * s.dv + col0;
 
     for (int e = tid; e < Np * SC_COLS; e += NT) {
         const int d = e / SC_COLS, c = e % SC_COLS;
-        St[c * KS + d] = (d < s.N && col0 + c < s.dv) ? S[(size_t)d * s.dv + col0 + c] : 0.f;
+        St[c * KS + d] = (d < N && col0 + c < s.dv) ? S[(size_t)d * s.dv + col0 + c] : 0.f;
     }
     for (int e = tid; e < 2 * SC_L * KS; e += NT) Cs[e] = 0.f;      // B and C: the filling stays zero
     for (int e = tid; e < SC_L * TS; e += NT) Ps[e] = 0.f;          // tiles above the diagonal stay zero
 
     // eight threads per token fetch its B and C (16 bytes at a time where NV > 0) and its x a chunk
     // ahead, into registers
-    const int ft = tid >> 3, sub = tid & 7, n4 = s.N >> 2;
+    const int ft = tid >> 3, sub = tid & 7, n4 = N >> 2;
     float4 rb[NV > 0 ? NV : 1], rc[NV > 0 ? NV : 1];
     float rx[4], rd = 0.f;
     auto fetch = [&](int c0) {
@@ -230,7 +232,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
     fetch(t0);
     for (int c0 = t0; c0 < t1; c0 += SC_L) {
         const int Lc = t1 - c0 < SC_L ? t1 - c0 : SC_L;
-        __syncthreads();                         // the chunk before is done with everything
+        lds_barrier();                           // the chunk before is done with everything
         if (NV > 0) {
 #pragma unroll
             for (int i = 0; i < NV; ++i) {
@@ -243,7 +245,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
         } else {
             const bool live = ft < Lc;
             const float* cr = conv + (size_t)(c0 + (live ? ft : 0)) * s.conv_width;
-            for (int e = sub; e < s.N; e += 8) {
+            for (int e = sub; e < N; e += 8) {
                 Bs[ft * KS + e] = live ? cr[b_col + e] : 0.f;
                 Cs[ft * KS + e] = live ? cr[c_col + e] : 0.f;
             }
@@ -268,7 +270,7 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
             }
         }
         if (c0 + SC_L < t1) fetch(c0 + SC_L);
-        __syncthreads();
+        lds_barrier();
         // scores of the chunk, decayed: the 16 x 16 tiles on and below the diagonal, handed out
         // over the waves
         for (int idx = wave; idx < (SC_L / 16) * (SC_L / 16 + 1) / 2; idx += NW) {
@@ -278,15 +280,17 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
             sc_floatx4_t acc = {0.f, 0.f, 0.f, 0.f};
             const float* ca = Cs + (ti * 16 + li) * KS + 4 * lg;
             const float* bb = Bs + (si * 16 + li) * KS + 4 * lg;
+            const int tr0 = ti * 16 + lg * 4, ss = si * 16 + li;
+            const double run_s = run[ss];
+            const float dt_s = dts[ss];
+            float e[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) e[r] = expf((float)(run[tr0 + r] - run_s)) * dt_s;   // s > t: not used
 #pragma unroll 4
             for (int d0 = 0; d0 < Np; d0 += 16)
                 acc = sc_mfma4(*(const float4*)(ca + d0), *(const float4*)(bb + d0), acc);
-            const int ss = si * 16 + li;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = ti * 16 + lg * 4 + r;
-                Ps[t * TS + ss] = ss <= t ? acc[r] * expf((float)(run[t] - run[ss])) * dts[ss] : 0.f;
-            }
+            for (int r = 0; r < 4; ++r) Ps[(tr0 + r) * TS + ss] = ss <= tr0 + r ? acc[r] * e[r] : 0.f;
         }
         // the state's share of y for the workgroup's columns: exp(L_t) (C S0)
         sc_floatx4_t num = {0.f, 0.f, 0.f, 0.f};
@@ -294,13 +298,16 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
         {
             const float* ca = Cs + (oti * 16 + li) * KS + 4 * lg;
             const float* sb = St + (oci * 16 + li) * KS + 4 * lg;
+            float e[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) e[r] = expf((float)run[oti * 16 + lg * 4 + r]);
 #pragma unroll 4
             for (int d0 = 0; d0 < Np; d0 += 16)
                 num = sc_mfma4(*(const float4*)(ca + d0), *(const float4*)(sb + d0), num);
 #pragma unroll
-            for (int r = 0; r < 4; ++r) num[r] *= expf((float)run[oti * 16 + lg * 4 + r]);
+            for (int r = 0; r < 4; ++r) num[r] *= e[r];
         }
-        __syncthreads();                         // Ps is whole, St has been read by every wave
+        lds_barrier();                           // Ps is whole, St has been read by every wave
         {
             const float* pa = Ps + (oti * 16 + li) * TS + 4 * lg;
             const float* xb = Xt + (oci * 16 + li) * TS + 4 * lg;
@@ -338,8 +345,8 @@ __global__ __launch_bounds__(SC_L * 8) void state_space_chunk_kernel(
             }
         }
     }
-    __syncthreads();
-    for (int e = tid; e < s.N * SC_COLS; e += NT) {
+    lds_barrier();
+    for (int e = tid; e < N * SC_COLS; e += NT) {
         const int d = e / SC_COLS, c = e % SC_COLS;
         if (col0 + c < s.dv) S[(size_t)d * s.dv + col0 + c] = St[c * KS + d];
     }
@@ -371,7 +378,7 @@ extern "C" int gfa_state_space_chunks_take(int N, int dv) {
     return N >= 1 && dv >= 1 && sc_fits(N, 32) ? 1 : 0;
 }
 
-template <int L, int NV>
+template <int L, int NV, int NC>
 static int sc_launch(const float* conv, const float* proj, const float* A_log, const float* dt_bias,
                      const float* skip, float* state, size_t slot_stride, const int* q_start,
                      const int* slots, float* out, const SSShape& s, int n_seqs, hipStream_t stream) {
@@ -379,14 +386,14 @@ static int sc_launch(const float* conv, const float* proj, const float* A_log, c
     if (bytes > 64 * 1024) {
         static bool allowed = false;
         if (!allowed) {
-            const hipError_t e = hipFuncSetAttribute((const void*)state_space_chunk_kernel<L, NV>,
+            const hipError_t e = hipFuncSetAttribute((const void*)state_space_chunk_kernel<L, NV, NC>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             if (e != hipSuccess) return (int)e;
             allowed = true;
         }
     }
     const int n_cols = (s.dv + SC_COLS - 1) / SC_COLS;
-    state_space_chunk_kernel<L, NV><<<n_cols * s.H * n_seqs, L * 8, bytes, stream>>>(
+    state_space_chunk_kernel<L, NV, NC><<<n_cols * s.H * n_seqs, L * 8, bytes, stream>>>(
         conv, proj, A_log, dt_bias, skip, state, slot_stride, q_start, slots, out, s, n_cols, n_seqs);
     return GFA_LAUNCH_RESULT();
 }
@@ -407,13 +414,15 @@ extern "C" int gfa_state_space_chunks(const float* conv, int conv_width, const f
     const bool vec = N % 4 == 0 && conv_width % 4 == 0 && (H * dv) % 4 == 0 && (size_t)conv % 16 == 0
         && N <= 256;
     const bool big = max_q_len > 32 && sc_fits(N, 64);
-#define SC_GO(NV) return big ? sc_launch<64, NV>(conv, proj, A_log, dt_bias, skip, state, slot_stride, q_start, \
-                                                 slots, out, s, n_seqs, stream) \
-                             : sc_launch<32, NV>(conv, proj, A_log, dt_bias, skip, state, slot_stride, q_start, \
-                                                 slots, out, s, n_seqs, stream)
-    if (!vec) SC_GO(0);
-    if (N <= 64) SC_GO(2);
-    if (N <= 128) SC_GO(4);
-    SC_GO(8);
+#define SC_GO(NV, NC) return big ? sc_launch<64, NV, NC>(conv, proj, A_log, dt_bias, skip, state, slot_stride, \
+                                                       q_start, slots, out, s, n_seqs, stream) \
+                                 : sc_launch<32, NV, NC>(conv, proj, A_log, dt_bias, skip, state, slot_stride, \
+                                                       q_start, slots, out, s, n_seqs, stream)
+    if (!vec) SC_GO(0, 0);
+    if (N == 64) SC_GO(2, 64);
+    if (N == 128) SC_GO(4, 128);
+    if (N <= 64) SC_GO(2, 0);
+    if (N <= 128) SC_GO(4, 0);
+    SC_GO(8, 0);
 #undef SC_GO
 }

@@ -239,7 +239,7 @@ def test_the_convolution_with_its_bias_from_a_column_on(K_, C, column, extra):
 
 
 @pytest.mark.parametrize("chunked", [0, 32, 64])
-@pytest.mark.parametrize("H,G,N,dv", [(6, 3, 24, 16), (1, 1, 12, 40), (4, 4, 6, 10), (8, 2, 128, 64), (2, 1, 136, 33),
+@pytest.mark.parametrize("H,G,N,dv", [(6, 3, 24, 16), (1, 1, 12, 40), (4, 4, 6, 10), (8, 2, 128, 64), (4, 2, 64, 48), (2, 1, 136, 33),
                                       (3, 1, 70, 144)])
 def test_the_cell_with_carried_state_token_by_token_and_in_chunks(H, G, N, dv, chunked):
     """Three sequences in scattered slots, fed in portions of unequal sizes (down to one and two
