@@ -1,2 +1,2 @@
 """Architectures this library knows.  Importing a module registers its architecture."""
-from . import bikadra, llama, nizedra, pigodra, refolix, vusenex  # noqa: F401
+from . import bikadra, llama, nizedra, pigodra, pitenex, refolix, vusenex  # noqa: F401

@@ -21,12 +21,14 @@ class NormSpec:
     kind "rms": a weight per element.  kind "rms_scalar": one stored number for all elements.
     kind "none": no norm at all; the rows are only handed on in the compute type (a sublayer
     that reads the residual stream itself).
-    kind "layer": the layer norm with a weight and no bias, ``(x - mean) / sqrt(var + eps) * w``
-    with the variance as the mean of the squared deviations."""
+    kind "layer": the layer norm with a weight, ``(x - mean) / sqrt(var + eps) * w``
+    with the variance as the mean of the squared deviations, and with ``bias`` a bias per element
+    that is added."""
     dim: int
     eps: float
     kind: str = "rms"
     weight_offset: float = 0.0
+    bias: bool = False
 
 
 @dataclass(frozen=True)
@@ -105,8 +107,10 @@ class NormedAttentionSpec:
     that all heads share (one for q, one for k), before they are rotated.  ``position`` rotates
     the first ``position.rotary_dim`` elements of every head (any layout and scaling of
     ``PositionSpec``).  score = (q . k) * scale, then ``softcap tanh(score / softcap)`` if
-    ``softcap``; ``window`` W: keys at distance < W only; ordinary softmax; values of
-    ``value_dim``."""
+    ``softcap``; ``window`` W: keys at distance < W only; ``chunk`` C: keys j of the query's own
+    chunk only, ``j // C == i // C``, chunks counted from the sequence's first token; ``sink``: the
+    softmax's denominator has one more term exp(sink_h), a learned number per head (not scaled,
+    without a value).  Values of ``value_dim``."""
     dim: int
     n_heads: int
     n_kv_heads: int
@@ -117,6 +121,8 @@ class NormedAttentionSpec:
     qk_norm_eps: Optional[float] = None
     softcap: Optional[float] = None
     window: Optional[int] = None
+    chunk: Optional[int] = None
+    sink: bool = False
     kind: str = "normed_attention"
 
 
@@ -131,8 +137,12 @@ class GatedDeltaSpec:
     dt_bias))`` per head; per head a float32 state ``S [key_dim, value_dim]``, zero at a
     sequence's start: ``S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q``.  Each head's
     o is divided by its root mean square (``eps``), times a weight of ``value_dim`` elements that
-    the heads share, times silu of a gate projection, then projected out.  The convolutions'
-    last ``conv_taps - 1`` inputs are part of the sequence's state."""
+    the heads share, times ``gate`` ("silu" or "sigmoid") of a gate projection, then projected out.
+    The convolutions' last ``conv_taps - 1`` inputs are part of the sequence's state.
+    ``decay_rank`` R (None: as above): a decay per head and key channel, ``g = exp(-exp(A_log_h)
+    softplus(w_a2 (w_a1 x) + dt_bias))`` with ``w_a1`` [R, dim] and ``n_heads * key_dim`` numbers of
+    ``w_a2`` and ``dt_bias``, acting on S's rows.  ``gate_rank``: the gate projection is a product of
+    two matrices with so many rows between them."""
     dim: int
     n_heads: int
     n_kv_heads: int
@@ -141,6 +151,9 @@ class GatedDeltaSpec:
     conv_taps: int
     eps: float
     unit_eps: float = 1e-6
+    gate: str = "silu"
+    decay_rank: Optional[int] = None
+    gate_rank: Optional[int] = None
     kind: str = "gated_delta"
 
 
@@ -173,11 +186,14 @@ class ParallelMixerSpec:
     """Several mixers side by side that read the same input: ``branches`` = ((name, spec), ...),
     each any mixer spec.  The result is the mean of the branches' results, each first divided
     by its root mean square over the model width (``eps`` inside the root) and multiplied by a
-    weight per element of its own (parameter ``<name>_out``).  Each branch keeps its own cache
+    weight per element of its own (parameter ``<name>_out``).  With ``scales``, one number per branch,
+    the result is instead the sum of the branches' results times their numbers, with no norm and
+    no weights (``eps`` is not used).  Each branch keeps its own cache
     (``cache.store.JointNeed``); a branch's parameters are named ``<name>.<parameter>``."""
     dim: int
     branches: Tuple[Tuple[str, object], ...]
-    eps: float
+    eps: Optional[float] = None
+    scales: Optional[Tuple[float, ...]] = None
     kind: str = "parallel"
 
 
@@ -311,7 +327,12 @@ class RoutedExpertsSpec:
     with the largest choice scores are.  Their weights are their ``s`` over the sum of the
     chosen ``s`` (plus ``weight_eps``).  ``shared_hidden`` > 0: one more expert of that inner
     size and the same form runs for every token, with weight one or, with ``shared_gate``,
-    ``sigmoid(w_sg x)`` (one number per token)."""
+    ``sigmoid(w_sg x)`` (one number per token).
+    ``identity``: so many further router outputs stand behind the experts' (the router, the
+    correction, the scores and the choice cover all of them); a token that chooses one adds its x
+    itself, times the weight.  ``activation`` "clamped_swish" (gated experts; see
+    ``GatedFeedForwardSpec``) clamps at ``limit`` in the experts and at ``shared_limit`` in the
+    shared expert."""
     dim: int
     n_experts: int
     top: int
@@ -326,6 +347,9 @@ class RoutedExpertsSpec:
     group_top: int = 1
     gated: bool = False
     shared_gate: bool = False
+    identity: int = 0
+    limit: Optional[float] = None
+    shared_limit: Optional[float] = None
     kind: str = "routed_experts"
 
 
@@ -393,10 +417,12 @@ class InputMixSpec:
 @dataclass(frozen=True)
 class GatedFeedForwardSpec:
     """w2( act(w1 x) * (w3 x) ) without biases (reference model.py:219-227); ``activation``
-    "silu" or "gelu_tanh"."""
+    "silu", "gelu_tanh", or "clamped_swish" with ``limit``: ``a sigmoid(1.702 a) (b + 1)`` in place
+    of ``act(w1 x) * (w3 x)``, with a = min(w1 x, limit) and b = w3 x clamped to -limit .. limit."""
     dim: int
     hidden: int
     activation: str = "silu"
+    limit: Optional[float] = None
     kind: str = "gated"
 
 
@@ -413,7 +439,10 @@ class LayerSpec:
     In the "hyper_connected" arrangement ``streams`` copies x_1 .. x_S stand in place of one
     stream (hyper-connections): a sublayer reads ``norm(sum_s in[s] x_s)`` and gives y, and all
     streams move at once, ``x_t <- sum_s mix[s, t] x_s + out[t] y``, with stored numbers ``in [S]``,
-    ``out [S]`` and ``mix [S, S]`` (from, to) per sublayer."""
+    ``out [S]`` and ``mix [S, S]`` (from, to) per sublayer.
+    In the "parallel" arrangement mixer and feed-forward read the same rows and join the stream
+    together, ``x <- x + result_scale * (mixer(norm(x)) + ffn(norm(x)))``; the norm is
+    ``mixer_norm``."""
     name: str
     mixer: object
     mixer_norm: NormSpec
@@ -442,6 +471,8 @@ class LayerSpec:
     # "post_norm": the stream's factor in the sum, and a weight per element on each result
     residual_scale: float = 1.0
     layer_scale: bool = False
+    # "parallel": a factor on what joins the stream
+    result_scale: float = 1.0
     mixer_scale_name: str = "mixer_scale"
     feed_forward_scale_name: str = "feed_forward_scale"
 

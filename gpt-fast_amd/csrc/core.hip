@@ -578,24 +578,31 @@ extern "C" int gfa_attention_generic(const void* q, const void* k_pages, const v
 }
 
 // --------------------------------------------------------------------------------------
-// gate: out[n, i] = act(gu[n, i]) * gu[n, I + i]; act 0 = silu (model.py:227), 1 = the tanh
-// form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
+// gate: out[n, i] = pair(gu[n, i], gu[n, I + i]) with pair(a, b) = act(a) * b; act 0 = silu
+// (model.py:227), 1 = the tanh form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))).  act 2
+// clamps both first, a <- min(a, limit), b <- min(max(b, -limit), limit), and gives
+// a sigmoid(1.702 a) (b + 1).
 template <int ACT>
-__device__ __forceinline__ float gate_act(float a) {
-    if (ACT == 0) return a / (1.f + expf(-a));
-    return 0.5f * a * (1.f + tanhf(0.7978845608028654f * (a + 0.044715f * a * a * a)));
+__device__ __forceinline__ float gate_pair(float a, float b, float limit) {
+    if (ACT == 0) return a / (1.f + expf(-a)) * b;
+    if (ACT == 2) {
+        a = fminf(a, limit);
+        b = fminf(fmaxf(b, -limit), limit);
+        return a / (1.f + expf(-1.702f * a)) * (b + 1.f);
+    }
+    return 0.5f * a * (1.f + tanhf(0.7978845608028654f * (a + 0.044715f * a * a * a))) * b;
 }
 
 template <typename T, int ACT>
 __global__ void gate_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int I,
-                                size_t total) {
+                                size_t total, float limit) {
     for (size_t e = blockIdx.x * (size_t)blockDim.x + threadIdx.x; e < total;
          e += (size_t)gridDim.x * blockDim.x) {
         const size_t n = e / I;
         const int i = (int)(e % I);
         const float a = load_as_float(gu + n * 2 * I + i);
         const float b = load_as_float(gu + n * 2 * I + I + i);
-        store_from_float(out + e, gate_act<ACT>(a) * b);
+        store_from_float(out + e, gate_pair<ACT>(a, b, limit));
     }
 }
 
@@ -603,7 +610,7 @@ __global__ void gate_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, i
 template <int ACT>
 __global__ __launch_bounds__(256) void gate_mul_bf16x8_kernel(const bf16_t* __restrict__ gu,
                                                               bf16_t* __restrict__ out, int I8,
-                                                              size_t total8) {
+                                                              size_t total8, float limit) {
     const size_t e = blockIdx.x * (size_t)256 + threadIdx.x;
     if (e >= total8) return;
     const size_t n = e / I8;
@@ -615,39 +622,40 @@ __global__ __launch_bounds__(256) void gate_mul_bf16x8_kernel(const bf16_t* __re
     bf16_t* oe = (bf16_t*)&o;
 #pragma unroll
     for (int j = 0; j < 8; ++j)
-        oe[j] = float_to_bf16(gate_act<ACT>(bf16_to_float(ae[j])) * bf16_to_float(be[j]));
+        oe[j] = float_to_bf16(gate_pair<ACT>(bf16_to_float(ae[j]), bf16_to_float(be[j]), limit));
     ((uint4*)out)[e] = o;
 }
 
 template <int ACT>
-static int launch_gate_mul(const void* gu, void* out, int n_rows, int I, int is_bf16,
+static int launch_gate_mul(const void* gu, void* out, int n_rows, int I, int is_bf16, float limit,
                            hipStream_t stream) {
     const size_t total = (size_t)n_rows * I;
     if (total == 0) return 0;
     if (is_bf16 && I % 8 == 0) {
         const size_t total8 = total / 8;
         gate_mul_bf16x8_kernel<ACT><<<(unsigned)((total8 + 255) / 256), 256, 0, stream>>>(
-            (const bf16_t*)gu, (bf16_t*)out, I / 8, total8);
+            (const bf16_t*)gu, (bf16_t*)out, I / 8, total8, limit);
         return GFA_LAUNCH_RESULT();
     }
     const int blocks = (int)((total + 255) / 256 < 65535 ? (total + 255) / 256 : 65535);
     if (is_bf16)
-        gate_mul_kernel<bf16_t, ACT><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I, total);
+        gate_mul_kernel<bf16_t, ACT><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I, total, limit);
     else
-        gate_mul_kernel<float, ACT><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)out, I, total);
+        gate_mul_kernel<float, ACT><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)out, I, total, limit);
     return GFA_LAUNCH_RESULT();
 }
 
-extern "C" int gfa_gate_mul(const void* gu, void* out, int n_rows, int I, int act, int is_bf16,
+extern "C" int gfa_gate_mul(const void* gu, void* out, int n_rows, int I, int act, float limit, int is_bf16,
                             hipStream_t stream) {
-    if (act == 0) return launch_gate_mul<0>(gu, out, n_rows, I, is_bf16, stream);
-    if (act == 1) return launch_gate_mul<1>(gu, out, n_rows, I, is_bf16, stream);
+    if (act == 0) return launch_gate_mul<0>(gu, out, n_rows, I, is_bf16, limit, stream);
+    if (act == 1) return launch_gate_mul<1>(gu, out, n_rows, I, is_bf16, limit, stream);
+    if (act == 2) return launch_gate_mul<2>(gu, out, n_rows, I, is_bf16, limit, stream);
     return (int)hipErrorInvalidValue;
 }
 
 extern "C" int gfa_silu_mul(const void* gu, void* out, int n_rows, int I, int is_bf16,
                             hipStream_t stream) {
-    return launch_gate_mul<0>(gu, out, n_rows, I, is_bf16, stream);
+    return launch_gate_mul<0>(gu, out, n_rows, I, is_bf16, 0.f, stream);
 }
 
 // --------------------------------------------------------------------------------------
@@ -1319,15 +1327,15 @@ extern "C" int gfa_gated_normed_add(float* res, const float* y, const float* gat
 }
 
 // --------------------------------------------------------------------------------------
-// Layer norm with a weight and no bias:
-//   out[i, :] = (x[r, :] - mean) * rsqrt(mean((x[r, :] - mean)^2) + eps) * w[:],  r = rows ? rows[i] : i
+// Layer norm with a weight and, if `bias` is given, a bias:
+//   out[i, :] = (x[r, :] - mean) * rsqrt(mean((x[r, :] - mean)^2) + eps) * w[:] + bias[:],  r = rows ? rows[i] : i
 // The variance is the mean of the squared deviations (a second pass over the row, which a
 // thread keeps in registers up to 256 * GN_MAX elements).  Float arithmetic, one rounding at
 // the store.
 template <typename T>
 __global__ __launch_bounds__(256) void layer_norm_kernel(
-        const float* __restrict__ x, const float* __restrict__ w, const int* __restrict__ rows,
-        T* __restrict__ out, int dim, float eps) {
+        const float* __restrict__ x, const float* __restrict__ w, const float* __restrict__ bias,
+        const int* __restrict__ rows, T* __restrict__ out, int dim, float eps) {
     __shared__ float scratch[16];
     const size_t r = rows ? (size_t)rows[blockIdx.x] : (size_t)blockIdx.x;
     const float* xr = x + r * dim;
@@ -1365,20 +1373,21 @@ __global__ __launch_bounds__(256) void layer_norm_kernel(
 #pragma unroll
         for (int j = 0; j < GN_MAX; ++j) {
             const int d = threadIdx.x + 256 * j;
-            if (d < dim) store_from_float(o + d, (held[j] - mean) * rs * w[d]);
+            if (d < dim) store_from_float(o + d, (held[j] - mean) * rs * w[d] + (bias ? bias[d] : 0.f));
         }
     } else {
-        for (int d = threadIdx.x; d < dim; d += 256) store_from_float(o + d, (xr[d] - mean) * rs * w[d]);
+        for (int d = threadIdx.x; d < dim; d += 256)
+            store_from_float(o + d, (xr[d] - mean) * rs * w[d] + (bias ? bias[d] : 0.f));
     }
 }
 
-extern "C" int gfa_layer_norm(const float* x, const float* w, const int* rows, void* out, int out_bf16,
-                              int n_rows, int dim, float eps, hipStream_t stream) {
+extern "C" int gfa_layer_norm(const float* x, const float* w, const float* bias, const int* rows, void* out,
+                              int out_bf16, int n_rows, int dim, float eps, hipStream_t stream) {
     if (n_rows <= 0) return 0;
     if (out_bf16)
-        layer_norm_kernel<bf16_t><<<n_rows, 256, 0, stream>>>(x, w, rows, (bf16_t*)out, dim, eps);
+        layer_norm_kernel<bf16_t><<<n_rows, 256, 0, stream>>>(x, w, bias, rows, (bf16_t*)out, dim, eps);
     else
-        layer_norm_kernel<float><<<n_rows, 256, 0, stream>>>(x, w, rows, (float*)out, dim, eps);
+        layer_norm_kernel<float><<<n_rows, 256, 0, stream>>>(x, w, bias, rows, (float*)out, dim, eps);
     return GFA_LAUNCH_RESULT();
 }
 
@@ -1639,28 +1648,51 @@ extern "C" int gfa_rotate_rows(float* x, int row_width, int off, int n_heads, in
 }
 
 // --------------------------------------------------------------------------------------
-// The gate over float sums, rounded once: out[n, i] = act(gu[n, i]) * gu[n, I + i] as
+// The gate over float sums, rounded once: out[n, i] = pair(gu[n, i], gu[n, I + i]) as
 // bfloat16, gu float [N, 2 I] (the sums of a product whose rows are the gate rows and then
-// the up rows).  act 0: silu, 1: gelu (tanh form).
+// the up rows).  act as above.
 template <int ACT>
 __global__ void gate_mul_sums_kernel(const float* __restrict__ gu, bf16_t* __restrict__ out, int I,
-                                     size_t total) {
+                                     size_t total, float limit) {
     for (size_t e = blockIdx.x * (size_t)blockDim.x + threadIdx.x; e < total;
          e += (size_t)gridDim.x * blockDim.x) {
         const size_t n = e / I;
         const int i = (int)(e % I);
-        out[e] = float_to_bf16(gate_act<ACT>(gu[n * 2 * I + i]) * gu[n * 2 * I + I + i]);
+        out[e] = float_to_bf16(gate_pair<ACT>(gu[n * 2 * I + i], gu[n * 2 * I + I + i], limit));
     }
 }
 
-extern "C" int gfa_gate_mul_sums(const float* gu, void* out, int n_rows, int I, int act,
+extern "C" int gfa_gate_mul_sums(const float* gu, void* out, int n_rows, int I, int act, float limit,
                                  hipStream_t stream) {
     const size_t total = (size_t)n_rows * I;
     if (total == 0) return 0;
     const int blocks = (int)((total + 255) / 256 < 65535 ? (total + 255) / 256 : 65535);
-    if (act == 0) gate_mul_sums_kernel<0><<<blocks, 256, 0, stream>>>(gu, (bf16_t*)out, I, total);
-    else if (act == 1) gate_mul_sums_kernel<1><<<blocks, 256, 0, stream>>>(gu, (bf16_t*)out, I, total);
+    if (act == 0) gate_mul_sums_kernel<0><<<blocks, 256, 0, stream>>>(gu, (bf16_t*)out, I, total, limit);
+    else if (act == 1) gate_mul_sums_kernel<1><<<blocks, 256, 0, stream>>>(gu, (bf16_t*)out, I, total, limit);
+    else if (act == 2) gate_mul_sums_kernel<2><<<blocks, 256, 0, stream>>>(gu, (bf16_t*)out, I, total, limit);
     else return (int)hipErrorInvalidValue;
+    return GFA_LAUNCH_RESULT();
+}
+
+// out[n, i] = x[n * x_stride + i] for i < width, rounded to T: columns of float rows as rows of
+// their own (the operand of a further product).
+template <typename T>
+__global__ void cast_columns_kernel(const float* __restrict__ x, long long x_stride, T* __restrict__ out,
+                                    int width, size_t total) {
+    for (size_t e = blockIdx.x * (size_t)blockDim.x + threadIdx.x; e < total;
+         e += (size_t)gridDim.x * blockDim.x) {
+        const size_t n = e / width;
+        store_from_float(out + e, x[n * x_stride + (e - n * width)]);
+    }
+}
+
+extern "C" int gfa_cast_columns(const float* x, long long x_stride, void* out, int n_rows, int width,
+                                int out_bf16, hipStream_t stream) {
+    const size_t total = (size_t)n_rows * width;
+    if (total == 0) return 0;
+    const int blocks = (int)((total + 255) / 256 < 65535 ? (total + 255) / 256 : 65535);
+    if (out_bf16) cast_columns_kernel<bf16_t><<<blocks, 256, 0, stream>>>(x, x_stride, (bf16_t*)out, width, total);
+    else cast_columns_kernel<float><<<blocks, 256, 0, stream>>>(x, x_stride, (float*)out, width, total);
     return GFA_LAUNCH_RESULT();
 }
 

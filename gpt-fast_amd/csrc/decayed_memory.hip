@@ -365,19 +365,20 @@ extern "C" int gfa_decayed_memory_chunks(const float* proj, const float* decay, 
 template <typename T>
 __global__ __launch_bounds__(1024) void row_norm_gate_kernel(
         const float* __restrict__ o, const float* __restrict__ weight, int weight_width,
-        const float* __restrict__ proj, int row_width, int g_off, T* __restrict__ y, int width,
-        int groups, int gate_act, float eps) {
+        const float* __restrict__ proj, int row_width, int g_off, T* __restrict__ out, long long out_stride,
+        int width, int groups, int gate_act, float eps) {
     __shared__ float scratch[16];
     const size_t t = blockIdx.x;
     const float* src = o + t * width;
     const float* gate = proj + t * row_width + g_off;
+    T* y = out + t * out_stride;
     if (groups == 1) {
         float ss = 0.f;
         for (int d = threadIdx.x; d < width; d += blockDim.x) ss = fmaf(src[d], src[d], ss);
         const float r = rsqrtf(block_sum(ss, scratch) / (float)width + eps);
         for (int d = threadIdx.x; d < width; d += blockDim.x) {
             const float g = gate[d], sg = 1.f / (1.f + expf(-g));
-            store_from_float(y + t * width + d, src[d] * r * (weight ? weight[d % weight_width] : 1.f)
+            store_from_float(y + d, src[d] * r * (weight ? weight[d % weight_width] : 1.f)
                                                 * (gate_act ? g * sg : sg));
         }
         return;
@@ -390,26 +391,26 @@ __global__ __launch_bounds__(1024) void row_norm_gate_kernel(
         const float r = rsqrtf(wave_sum(ss) / (float)part + eps);
         for (int d = base + lane; d < base + part; d += 64) {
             const float g = gate[d], sg = 1.f / (1.f + expf(-g));
-            store_from_float(y + t * width + d, src[d] * r * (weight ? weight[d % weight_width] : 1.f)
+            store_from_float(y + d, src[d] * r * (weight ? weight[d % weight_width] : 1.f)
                                                 * (gate_act ? g * sg : sg));
         }
     }
 }
 
 extern "C" int gfa_row_norm_gate(const float* o, const float* weight, int weight_width,
-                                 const float* proj, int row_width, int g_off, void* y, int y_bf16,
-                                 int n_tokens, int width, int groups, int gate_act, float eps,
+                                 const float* proj, int row_width, int g_off, void* y, long long y_stride,
+                                 int y_bf16, int n_tokens, int width, int groups, int gate_act, float eps,
                                  hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (groups < 1 || width % groups || (weight && (weight_width < 1 || width % weight_width)))
+    if (groups < 1 || width % groups || y_stride < width || (weight && (weight_width < 1 || width % weight_width)))
         return (int)hipErrorInvalidValue;
     const int threads = width > 1024 ? 1024 : 256;       // an element or a few per thread
     if (y_bf16)
         row_norm_gate_kernel<bf16_t><<<n_tokens, threads, 0, stream>>>(
-            o, weight, weight_width, proj, row_width, g_off, (bf16_t*)y, width, groups, gate_act, eps);
+            o, weight, weight_width, proj, row_width, g_off, (bf16_t*)y, y_stride, width, groups, gate_act, eps);
     else
         row_norm_gate_kernel<float><<<n_tokens, threads, 0, stream>>>(
-            o, weight, weight_width, proj, row_width, g_off, (float*)y, width, groups, gate_act, eps);
+            o, weight, weight_width, proj, row_width, g_off, (float*)y, y_stride, width, groups, gate_act, eps);
     return GFA_LAUNCH_RESULT();
 }
 

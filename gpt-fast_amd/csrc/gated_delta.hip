@@ -9,6 +9,9 @@
 //     beta = sigmoid(b')      g = exp(-exp(A_log_h) softplus(a' + dt_bias_h))
 //     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
 //
+// With a decay per key channel a' and dt_bias are numbers per (head, channel) and g is a diagonal:
+// row d of S is multiplied by g_d.
+//
 // Head h of v, beta, g and o uses head h / (H / G) of q and k.  Everything here is float
 // arithmetic.  One slot's state: S [H][dk][dv], then the convolutions' tails [K - 1][C], oldest
 // first, C = 2 G dk + H dv channels in the order q, k, v.  The convolutions are short_conv.hip's.
@@ -25,6 +28,8 @@ struct GDShape {
     int conv_width;                     // floats per row of the convolved q, k, v
     int row_width;                      // floats per row of proj
     int b_off, a_off;                   // columns of beta's and the decay's pre-activations in proj
+    const float* decays;                // a decay per channel: rows of its pre-activations [.., H dk], else null
+    int decay_width;                    // floats per row of decays
     float q_scale, unit_eps;
 };
 
@@ -34,14 +39,17 @@ struct GDShape {
 // over the thread's rows and one exchange through shared memory; with rk, rq the unit norms'
 // factors:  u = beta (v - rk a),  S = Sg + rk k' u^T,  o = rq (b + rk (k'.q') u),
 // which is S^T q after the write.  q', k' and the exchange buffer alternate between two
-// copies, so a token costs two barriers; the next token's values are fetched meanwhile.
-template <int RPT>
+// copies, so a token costs two barriers; the next token's values are fetched meanwhile.  CHAN: a
+// decay per key channel, worked out once per workgroup and element by the threads that fetch q
+// and k.
+template <int RPT, bool CHAN>
 __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
         const float* __restrict__ conv, const float* __restrict__ proj,
         const float* __restrict__ A_log, const float* __restrict__ dt_bias,
         float* __restrict__ state, size_t slot_stride, const int* __restrict__ q_start,
         const int* __restrict__ slots, float* __restrict__ out, GDShape s) {
     __shared__ float qs[2][RPT * GD_GROUPS], ks[2][RPT * GD_GROUPS];
+    __shared__ float gs[2][CHAN ? RPT * GD_GROUPS : 1];
     __shared__ float red[2][5][GD_GROUPS][GD_COLS];
     const int tid = threadIdx.x, c = tid % GD_COLS, g = tid / GD_COLS;
     const int col = blockIdx.x * GD_COLS + c;
@@ -50,7 +58,7 @@ __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
     const int t0 = q_start[b], t1 = q_start[b + 1];
     float* const S = state + (size_t)slots[b] * slot_stride + (size_t)h * s.dk * s.dv;
     const bool col_ok = col < s.dv;
-    const float rate = expf(A_log[h]), bias = dt_bias[h];
+    const float rate = expf(A_log[h]), bias = CHAN ? 0.f : dt_bias[h];
     const int q_col = kvh * s.dk, k_col = s.G * s.dk + kvh * s.dk, v_col = 2 * s.G * s.dk + h * s.dv;
     constexpr int EPT = (RPT * GD_GROUPS + GD_THREADS - 1) / GD_THREADS;   // elements of q a thread fetches
 
@@ -60,7 +68,7 @@ __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
         const int row = g + r * GD_GROUPS;
         Sreg[r] = (col_ok && row < s.dk) ? S[(size_t)row * s.dv + col] : 0.f;
     }
-    float nq[EPT], nk[EPT], nv = 0.f, nb = 0.f, na = 0.f;
+    float nq[EPT], nk[EPT], nz[EPT], nv = 0.f, nb = 0.f, na = 0.f;
     auto fetch = [&](int t) {
         const float* cr = conv + (size_t)t * s.conv_width;
 #pragma unroll
@@ -68,11 +76,13 @@ __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
             const int e = tid + i * GD_THREADS;
             nq[i] = e < s.dk ? cr[q_col + e] : 0.f;
             nk[i] = e < s.dk ? cr[k_col + e] : 0.f;
+            if (CHAN)
+                nz[i] = e < s.dk ? s.decays[(size_t)t * s.decay_width + h * s.dk + e] + dt_bias[h * s.dk + e] : 0.f;
         }
         nv = col_ok ? cr[v_col + col] : 0.f;
         const float* pr = proj + (size_t)t * s.row_width;
         nb = pr[s.b_off + h];
-        na = pr[s.a_off + h];
+        if (!CHAN) na = pr[s.a_off + h];
     };
     if (t0 < t1) fetch(t0);
     for (int t = t0; t < t1; ++t) {
@@ -83,11 +93,12 @@ __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
             if (e < RPT * GD_GROUPS) {
                 qs[p][e] = nq[i];
                 ks[p][e] = nk[i];
+                if (CHAN) gs[p][e] = expf(-rate * gd_softplus(nz[i]));
             }
         }
         const float v = nv;
         const float beta = 1.f / (1.f + expf(-nb));
-        const float decay = expf(-rate * gd_softplus(na + bias));
+        const float decay = CHAN ? 0.f : expf(-rate * gd_softplus(na + bias));
         if (t + 1 < t1) fetch(t + 1);
         __syncthreads();
         float pa = 0.f, pb = 0.f, kk = 0.f, qq = 0.f, kq = 0.f;
@@ -95,7 +106,7 @@ __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
         for (int r = 0; r < RPT; ++r) {
             const int e = g + r * GD_GROUPS;
             const float ke = ks[p][e], qe = qs[p][e];
-            Sreg[r] *= decay;
+            Sreg[r] *= CHAN ? gs[p][e] : decay;
             pa = fmaf(Sreg[r], ke, pa);
             pb = fmaf(Sreg[r], qe, pb);
             kk = fmaf(ke, ke, kk);
@@ -135,25 +146,30 @@ __global__ __launch_bounds__(GD_THREADS) void gated_delta_scan_kernel(
 }
 
 extern "C" int gfa_gated_delta_scan(const float* conv, int conv_width, const float* proj, int row_width,
-                                    int b_off, int a_off, const float* A_log, const float* dt_bias,
+                                    int b_off, int a_off, const float* decays, int decay_width,
+                                    const float* A_log, const float* dt_bias,
                                     float* state, size_t slot_stride, const int* q_start,
                                     const int* slots, float* out, int n_seqs, int H, int G, int dk,
                                     int dv, float q_scale, float unit_eps, hipStream_t stream) {
     if (n_seqs <= 0) return 0;
     if (dk < 1 || dk > 64 * GD_GROUPS || H < 1 || H > 65535 || G < 1 || H % G || n_seqs > 65535 ||
-            conv_width < 2 * G * dk + H * dv || b_off + H > row_width || a_off + H > row_width)
+            conv_width < 2 * G * dk + H * dv || b_off + H > row_width || (!decays && a_off + H > row_width) ||
+            (decays && decay_width < H * dk))
         return (int)hipErrorInvalidValue;
-    GDShape s{H, G, dk, dv, conv_width, row_width, b_off, a_off, q_scale, unit_eps};
+    GDShape s{H, G, dk, dv, conv_width, row_width, b_off, a_off, decays, decay_width, q_scale, unit_eps};
     dim3 grid((dv + GD_COLS - 1) / GD_COLS, H, n_seqs);
     const int rpt = (dk + GD_GROUPS - 1) / GD_GROUPS;
-#define GD_LAUNCH(R) gated_delta_scan_kernel<R><<<grid, GD_THREADS, 0, stream>>>( \
-        conv, proj, A_log, dt_bias, state, slot_stride, q_start, slots, out, s)
+#define GD_ARGS <<<grid, GD_THREADS, 0, stream>>>(conv, proj, A_log, dt_bias, state, slot_stride, q_start, \
+                                                  slots, out, s)
+#define GD_LAUNCH(R) do { if (decays) gated_delta_scan_kernel<R, true>GD_ARGS; \
+                          else gated_delta_scan_kernel<R, false>GD_ARGS; } while (0)
     if (rpt <= 4) GD_LAUNCH(4);
     else if (rpt <= 8) GD_LAUNCH(8);
     else if (rpt <= 16) GD_LAUNCH(16);
     else if (rpt <= 32) GD_LAUNCH(32);
     else GD_LAUNCH(64);
 #undef GD_LAUNCH
+#undef GD_ARGS
     return GFA_LAUNCH_RESULT();
 }
 
@@ -509,7 +525,7 @@ extern "C" int gfa_gated_delta_chunks(const float* conv, int conv_width, const f
             conv_width < 2 * G * dk + H * dv || b_off + H > row_width || a_off + H > row_width ||
             !gfa_gated_delta_chunks_take(dk, dv))
         return (int)hipErrorInvalidValue;
-    GDShape s{H, G, dk, dv, conv_width, row_width, b_off, a_off, q_scale, unit_eps};
+    GDShape s{H, G, dk, dv, conv_width, row_width, b_off, a_off, nullptr, 0, q_scale, unit_eps};
     dim3 grid((dv + GC_COLS - 1) / GC_COLS, H, n_seqs);
     // 16-byte loads of q and k where every row and head starts at a multiple of four floats
     const bool vec = dk % 4 == 0 && conv_width % 4 == 0 && (size_t)conv % 16 == 0 && dk <= 256;

@@ -13,6 +13,10 @@
 // chain of multiply-adds over its own inputs, so a token's result does not depend on what
 // else the step holds.  These kernels serve the float32 engine and the steps of few rows;
 // the weights of an expert are stacked: W_up [E, F, D], W_down [E, D, F].
+//
+// Identity experts: the router may have more outputs than there are stacked experts; a chosen
+// index of E or more stands for y = x itself.  Its pair takes part in no product, and the kernels
+// that add up a token's pairs add weight * x in its place.
 #include "common.h"
 
 #define RE_MAX_PER_LANE 16          // experts per lane of the router's wave: E <= 1024
@@ -143,6 +147,13 @@ extern "C" int gfa_route(const float* z, long long z_stride, int n_tokens, int E
     return GFA_LAUNCH_RESULT();
 }
 
+// the gate of clamped experts: a <- min(a, limit), b <- b clamped to -limit .. limit, a sigmoid(1.702 a) (b + 1)
+__device__ __forceinline__ float re_clamped_pair(float a, float b, float limit) {
+    a = fminf(a, limit);
+    b = fminf(fmaxf(b, -limit), limit);
+    return a / (1.f + expf(-1.702f * a)) * (b + 1.f);
+}
+
 // 0 silu, 1 gelu (tanh form), 3 gelu (exact); the numbers of ops.kernels.ACTIVATIONS
 __device__ __forceinline__ float re_activation(float z, int act) {
     if (act == 0) return z / (1.f + expf(-z));
@@ -192,14 +203,16 @@ __device__ __forceinline__ float re_row_dot(const T* __restrict__ w, const float
 #define RE_THREADS 256
 #define RE_ROWS 16                  // weight rows per workgroup: four per wave
 
-// h[pair, f] = act(W_up[e(pair)][f, :] . x[token(pair), :]);  grid (F / RE_ROWS, pairs)
+// h[pair, f] = act(W_up[e(pair)][f, :] . x[token(pair), :]);  grid (F / RE_ROWS, pairs).  gated 2: the
+// clamped gate.  A pair of an identity expert (e >= E) has no h.
 template <typename T>
 __global__ __launch_bounds__(RE_THREADS) void expert_up_kernel(
         const T* __restrict__ x, const T* __restrict__ w_up, const int* __restrict__ chosen,
-        T* __restrict__ h, int top, int D, int F, int act, int gated) {
+        T* __restrict__ h, int top, int D, int F, int E, int act, int gated, float limit) {
     extern __shared__ float re_x[];
     const int pair = blockIdx.y, n = pair / top;
     const int e = chosen[pair];
+    if (e >= E) return;                                // the whole workgroup
     for (int d = threadIdx.x; d < D; d += RE_THREADS) re_x[d] = load_as_float(x + (size_t)n * D + d);
     __syncthreads();
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -207,8 +220,13 @@ __global__ __launch_bounds__(RE_THREADS) void expert_up_kernel(
     for (int r = wave; r < RE_ROWS; r += RE_THREADS / 64) {
         const int f = blockIdx.x * RE_ROWS + r;
         if (f >= F) break;
-        float v = re_activation(re_row_dot<T>(w + (size_t)f * D, re_x, D, lane), act);
-        if (gated) v *= re_row_dot<T>(w + (size_t)(F + f) * D, re_x, D, lane);
+        float v = re_row_dot<T>(w + (size_t)f * D, re_x, D, lane);
+        if (gated == 2) {
+            v = re_clamped_pair(v, re_row_dot<T>(w + (size_t)(F + f) * D, re_x, D, lane), limit);
+        } else {
+            v = re_activation(v, act);
+            if (gated) v *= re_row_dot<T>(w + (size_t)(F + f) * D, re_x, D, lane);
+        }
         if (lane == 0) store_from_float(h + (size_t)pair * F + f, v);
     }
 }
@@ -217,12 +235,12 @@ __global__ __launch_bounds__(RE_THREADS) void expert_up_kernel(
 template <typename T>
 __global__ __launch_bounds__(RE_THREADS) void expert_down_kernel(
         const T* __restrict__ h, const T* __restrict__ w_down, const int* __restrict__ chosen,
-        const float* __restrict__ weights, float* __restrict__ y, int top, int D, int F,
-        int accumulate) {
+        const float* __restrict__ weights, const T* __restrict__ x, float* __restrict__ y, int top, int D,
+        int F, int E, int accumulate) {
     extern __shared__ float re_h[];                    // [top][F]
     const int n = blockIdx.y;
     for (int i = threadIdx.x; i < top * F; i += RE_THREADS)
-        re_h[i] = load_as_float(h + (size_t)n * top * F + i);
+        re_h[i] = chosen[(size_t)n * top + i / F] < E ? load_as_float(h + (size_t)n * top * F + i) : 0.f;
     __syncthreads();
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     for (int r = wave; r < RE_ROWS; r += RE_THREADS / 64) {
@@ -231,7 +249,8 @@ __global__ __launch_bounds__(RE_THREADS) void expert_down_kernel(
         float acc = 0.f;
         for (int k = 0; k < top; ++k) {
             const int e = chosen[(size_t)n * top + k];
-            const float v = re_row_dot<T>(w_down + ((size_t)e * D + c) * F, re_h + (size_t)k * F, F, lane);
+            const float v = e < E ? re_row_dot<T>(w_down + ((size_t)e * D + c) * F, re_h + (size_t)k * F, F, lane)
+                                  : load_as_float(x + (size_t)n * D + c);
             acc = fmaf(weights[(size_t)n * top + k], v, acc);
         }
         if (lane == 0) {
@@ -243,10 +262,10 @@ __global__ __launch_bounds__(RE_THREADS) void expert_down_kernel(
 
 extern "C" int gfa_experts_few_rows(const void* x, const void* w_up, const void* w_down,
                                     const int* chosen, const float* weights, void* h, float* y,
-                                    int n_tokens, int top, int D, int F, int act, int gated,
-                                    int accumulate, int is_bf16, hipStream_t stream) {
+                                    int n_tokens, int top, int D, int F, int E, int act, int gated,
+                                    float limit, int accumulate, int is_bf16, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (top <= 0 || D <= 0 || F <= 0 || (act != 0 && act != 1 && act != 3) || n_tokens * (long long)top > 65535
+    if (top <= 0 || D <= 0 || F <= 0 || E <= 0 || (act != 0 && act != 1 && act != 3) || n_tokens * (long long)top > 65535
             || n_tokens > 65535)
         return (int)hipErrorInvalidValue;
     const size_t up_lds = sizeof(float) * (size_t)D, down_lds = sizeof(float) * (size_t)top * F;
@@ -254,14 +273,14 @@ extern "C" int gfa_experts_few_rows(const void* x, const void* w_up, const void*
     dim3 up_grid((F + RE_ROWS - 1) / RE_ROWS, n_tokens * top), down_grid((D + RE_ROWS - 1) / RE_ROWS, n_tokens);
     if (is_bf16) {
         expert_up_kernel<bf16_t><<<up_grid, RE_THREADS, up_lds, stream>>>(
-            (const bf16_t*)x, (const bf16_t*)w_up, chosen, (bf16_t*)h, top, D, F, act, gated);
+            (const bf16_t*)x, (const bf16_t*)w_up, chosen, (bf16_t*)h, top, D, F, E, act, gated, limit);
         expert_down_kernel<bf16_t><<<down_grid, RE_THREADS, down_lds, stream>>>(
-            (const bf16_t*)h, (const bf16_t*)w_down, chosen, weights, y, top, D, F, accumulate);
+            (const bf16_t*)h, (const bf16_t*)w_down, chosen, weights, (const bf16_t*)x, y, top, D, F, E, accumulate);
     } else {
         expert_up_kernel<float><<<up_grid, RE_THREADS, up_lds, stream>>>(
-            (const float*)x, (const float*)w_up, chosen, (float*)h, top, D, F, act, gated);
+            (const float*)x, (const float*)w_up, chosen, (float*)h, top, D, F, E, act, gated, limit);
         expert_down_kernel<float><<<down_grid, RE_THREADS, down_lds, stream>>>(
-            (const float*)h, (const float*)w_down, chosen, weights, y, top, D, F, accumulate);
+            (const float*)h, (const float*)w_down, chosen, weights, (const float*)x, y, top, D, F, E, accumulate);
     }
     return GFA_LAUNCH_RESULT();
 }
@@ -367,7 +386,7 @@ extern "C" int gfa_gather_pairs_padded(const void* x, const int* order, const in
 }
 
 // padded[p] = chosen[p] * cap + place[p] - offsets[chosen[p]]: where pair p's row lies when every
-// expert's share is padded to `cap` rows
+// expert's share is padded to `cap` rows (an identity expert's pair: anywhere, it is never read)
 __global__ void padded_places_kernel(const int* __restrict__ place, const int* __restrict__ chosen,
                                      const int* __restrict__ offsets, int* __restrict__ padded,
                                      int n_pairs, int cap) {
@@ -385,37 +404,44 @@ extern "C" int gfa_padded_places(const int* place, const int* chosen, const int*
     return GFA_LAUNCH_RESULT();
 }
 
-// y[n, :] (+)= sum_k weight[n, k] ys[place[n top + k], :], in the order of the choice
-template <typename T>
+// y[n, :] (+)= sum_k weight[n, k] ys[place[n top + k], :], in the order of the choice; with `chosen`,
+// a pair whose expert is E or more adds weight * x[n, :] instead
+template <typename T, typename X>
 __global__ void combine_pairs_kernel(const T* __restrict__ ys, const int* __restrict__ place,
-                                     const float* __restrict__ weights, float* __restrict__ y,
+                                     const float* __restrict__ weights, const int* __restrict__ chosen,
+                                     int E, const X* __restrict__ x, float* __restrict__ y,
                                      int top, int D, int accumulate) {
     const int n = blockIdx.x;
     for (int d = blockIdx.y * blockDim.x + threadIdx.x; d < D; d += gridDim.y * blockDim.x) {
         float acc = 0.f;
-        for (int k = 0; k < top; ++k)
-            acc = fmaf(weights[(size_t)n * top + k],
-                       load_as_float(ys + (size_t)place[(size_t)n * top + k] * D + d), acc);
+        for (int k = 0; k < top; ++k) {
+            const size_t p = (size_t)n * top + k;
+            const float v = chosen && chosen[p] >= E ? load_as_float(x + (size_t)n * D + d)
+                                                     : load_as_float(ys + (size_t)place[p] * D + d);
+            acc = fmaf(weights[p], v, acc);
+        }
         float* o = y + (size_t)n * D + d;
         *o = accumulate ? *o + acc : acc;
     }
 }
 
-extern "C" int gfa_combine_pairs(const void* ys, const int* place, const float* weights, float* y,
-                                 int n_tokens, int top, int D, int accumulate, int is_bf16,
-                                 hipStream_t stream) {
+extern "C" int gfa_combine_pairs(const void* ys, const int* place, const float* weights, const int* chosen,
+                                 int E, const void* x, int x_bf16, float* y, int n_tokens, int top, int D,
+                                 int accumulate, int is_bf16, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
+    if (chosen && !x) return (int)hipErrorInvalidValue;
     // few tokens: a row's elements are spread over several workgroups
     int parts = (D + 255) / 256;
     if (parts > 32) parts = 32;
     if (n_tokens >= 1024) parts = 1;
     dim3 grid(n_tokens, parts);
-    if (is_bf16)
-        combine_pairs_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)ys, place, weights, y,
-                                                               top, D, accumulate);
-    else
-        combine_pairs_kernel<float><<<grid, 256, 0, stream>>>((const float*)ys, place, weights, y,
-                                                              top, D, accumulate);
+#define CP_GO(T, X) combine_pairs_kernel<T, X><<<grid, 256, 0, stream>>>( \
+        (const T*)ys, place, weights, chosen, E, (const X*)x, y, top, D, accumulate)
+    if (is_bf16 && x_bf16) CP_GO(bf16_t, bf16_t);
+    else if (is_bf16) CP_GO(bf16_t, float);
+    else if (x_bf16) CP_GO(float, bf16_t);
+    else CP_GO(float, float);
+#undef CP_GO
     return GFA_LAUNCH_RESULT();
 }
 

@@ -2,7 +2,8 @@
 // the softmax, and whose keys and values may have different sizes; all arithmetic in float.
 //
 // For the token at position i of a sequence, head h (kv head g = h / (H / G)) and key j with
-// max(0, i - window + 1) <= j <= i (window 0: from 0):
+// max(0, i - window + 1) <= j <= i (window 0: from 0), and with a chunk size C also floor(i / C) =
+// floor(j / C):
 //     s_h(j) = (q_h . k_g(j)) * scale * temperature[h]                  (temperature optional)
 //     s_h(j) = softcap * tanh(s_h(j) / softcap)                         (softcap > 0)
 //     s_h(j) = s_h(j) + bias[row(i - j), h]                             (bias optional)
@@ -10,8 +11,9 @@
 //     z_h(j) = sum_h' talk[h, h'] s_h'(j)                               (talk optional)
 //     out_h  = sum_j softmax_j(z_h)(j) v_g(j)
 //     out_h  = out_h sigmoid(gate[token, h])                            (gate optional)
-// With a sink the softmax's denominator has one more term, exp(0): a key of score zero that
-// carries no value (the running maximum starts at 0 and the running sum at 1).
+// With a sink the softmax's denominator has one more term, exp(z): a key of score z that carries
+// no value (the running maximum starts at z and the running sum at 1); z is 0, or a number per
+// head.  The result may be multiplied by a constant (out_factor) before it is rounded.
 // row(n) = lookup[n] for n < n_lookup, else bias_rows - 1 (the host fills the lookup table).
 //
 // The cache keeps keys and values in the orders of common.h (key_offset, value_offset) with
@@ -33,9 +35,22 @@ struct SAShape {
     float scale, softcap;
     int bias_rows, n_lookup;
     int sink;
+    const float* sinks;                          // a sink's score per head, or null: 0
+    int chunk;                                   // 0: none
+    float out_factor;
     const float* gate;                           // a row of pre-activations per token, or null
     long long gate_tok;                          // floats from one token's row to the next
 };
+
+// the first key that the query at `pos` sees
+__device__ __forceinline__ int sa_first_key(int pos, int window, int chunk) {
+    int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    if (chunk > 0) {
+        const int start = pos - pos % chunk;
+        lo = start > lo ? start : lo;
+    }
+    return lo;
+}
 
 template <typename T> struct Pack8;
 template <> struct Pack8<bf16_t> {
@@ -79,7 +94,7 @@ __global__ __launch_bounds__(SA_THREADS) void scored_attention_kernel(
     const int n = blockIdx.x, h0 = blockIdx.y * HB;
     const int pos = tok_pos[n];
     const int* pages = table + (size_t)tok_seq[n] * s.table_stride;
-    const int lo = (s.window > 0 && pos - s.window + 1 > 0) ? pos - s.window + 1 : 0;
+    const int lo = sa_first_key(pos, s.window, s.chunk);
     const int per_group = s.H / s.G;
 
     for (int e = threadIdx.x; e < nh * s.hd; e += SA_THREADS) {
@@ -90,7 +105,8 @@ __global__ __launch_bounds__(SA_THREADS) void scored_attention_kernel(
     float m[HPW], l[HPW], acc[HPW][VPT];
 #pragma unroll
     for (int i = 0; i < HPW; ++i) {
-        m[i] = s.sink ? 0.f : -INFINITY;
+        const int hs = h0 + wave + SA_WAVES * i;
+        m[i] = s.sink ? (s.sinks && hs < s.H ? s.sinks[hs] : 0.f) : -INFINITY;
         l[i] = s.sink ? 1.f : 0.f;
 #pragma unroll
         for (int e = 0; e < VPT; ++e) acc[i][e] = 0.f;
@@ -200,7 +216,7 @@ __global__ __launch_bounds__(SA_THREADS) void scored_attention_kernel(
 #pragma unroll
         for (int e = 0; e < VPT; ++e) {
             const int d = lane + 64 * e;
-            if (d < s.vd) store_from_float(o + d, acc[i][e] / l[i] * open);
+            if (d < s.vd) store_from_float(o + d, acc[i][e] / l[i] * open * s.out_factor);
         }
     }
 }
@@ -257,8 +273,8 @@ extern "C" int gfa_scored_attention(const void* q, const void* k_pages, const vo
                                     const int* tok_seq, const int* tok_pos, const int* table,
                                     int table_stride, const float* temperature, const float* bias,
                                     const int* lookup, const float* talk, const float* r1,
-                                    const float* r2, int sink, void* out, int n_tokens,
-                                    int H, int G, int hd, int vd, long long q_tok, long long q_head,
+                                    const float* r2, int sink, const float* sinks, int chunk,
+                                    float out_factor, void* out, int n_tokens, int H, int G, int hd, int vd, long long q_tok, long long q_head,
                                     long long o_tok, long long o_head, float scale, float softcap,
                                     int bias_rows, int n_lookup, int window, const float* gate,
                                     long long gate_tok, int is_bf16, hipStream_t stream) {
@@ -266,7 +282,7 @@ extern "C" int gfa_scored_attention(const void* q, const void* k_pages, const vo
     if (G <= 0 || H % G || hd <= 0 || vd <= 0 || vd > 512) return (int)hipErrorInvalidValue;
     if ((r1 == nullptr) != (r2 == nullptr)) return (int)hipErrorInvalidValue;
     SAShape s{H, G, hd, vd, q_tok, q_head, o_tok, o_head, table_stride, window, scale, softcap,
-              bias_rows, n_lookup, sink ? 1 : 0, gate, gate_tok};
+              bias_rows, n_lookup, sink ? 1 : 0, sinks, chunk, out_factor, gate, gate_tok};
     if (is_bf16)
         return sa_dispatch<bf16_t>(q, k_pages, v_pages, tok_seq, tok_pos, table, temperature, bias,
                                    lookup, talk, r1, r2, out, n_tokens, s, stream);
@@ -379,9 +395,9 @@ __global__ __launch_bounds__(MAXT) void scored_attention_mfma_kernel(
         head = g * gs + hg;
     }
     const int pos = spos + tok;
-    const int lo = (s.window > 0 && pos - s.window + 1 > 0) ? pos - s.window + 1 : 0;
+    const int lo = sa_first_key(pos, s.window, s.chunk);
     const int pos_max = spos + tok_hi;
-    const int lo_min = (s.window > 0 && spos + tok_lo - s.window + 1 > 0) ? spos + tok_lo - s.window + 1 : 0;
+    const int lo_min = sa_first_key(spos + tok_lo, s.window, s.chunk);
     const int last_key = spos + q_len - 1;             // the newest key the cache holds of this sequence
 
     // with a mix the small tables live in shared memory (the workgroup walks many key blocks
@@ -418,10 +434,10 @@ __global__ __launch_bounds__(MAXT) void scored_attention_mfma_kernel(
     sa_floatx4_t o[DVT];
 #pragma unroll
     for (int dt = 0; dt < DVT; ++dt) o[dt] = sa_floatx4_t{0.f, 0.f, 0.f, 0.f};
-    // a sink is one more key of score zero without a value: the maximum starts at 0 and the
-    // sum at 1 (once per row: in one lane group, and in the first wave of a tile's waves)
+    // a sink is one more key without a value: the maximum starts at its score (in units of log 2)
+    // and the sum at 1 (once per row: in one lane group, and in the first wave of a tile's waves)
     const bool sink_here = s.sink && (!SPLIT || wave == 0);
-    float m = sink_here ? 0.f : -INFINITY, l = (sink_here && lg == 0) ? 1.f : 0.f;
+    float m = sink_here ? (s.sinks ? s.sinks[head] * 1.4426950408889634f : 0.f) : -INFINITY, l = (sink_here && lg == 0) ? 1.f : 0.f;
     const float r1h = r1 ? r1[head] : 0.f, r2h = r1 ? r2[head] : 0.f;
 
     // SPLIT: the waves of a workgroup share one tile of rows and take its key blocks in turn
@@ -573,7 +589,7 @@ __global__ __launch_bounds__(MAXT) void scored_attention_mfma_kernel(
                         o[dt][j] = fmaf(theirs[32 + (dt * 16 + lg * 4 + j) * 16 + li], f, o[dt][j]);
         }
     }
-    float inv = l > 0.f ? 1.f / l : 0.f;
+    float inv = l > 0.f ? s.out_factor / l : 0.f;
     if (s.gate) inv /= 1.f + expf(-s.gate[(size_t)(q0 + tok) * s.gate_tok + head]);
     if (!row_ok) return;
     bf16_t* orow = out + (size_t)(q0 + tok) * s.o_tok + (size_t)head * s.o_head;
@@ -663,7 +679,7 @@ extern "C" int gfa_scored_attention_mfma(const void* q, const void* k_pages, con
                                          int table_stride, const float* temperature,
                                          const float* bias, const int* lookup, const float* talk,
                                          const float* r1, const float* r2, int sink,
-                                         void* out, int n_seqs, int max_q_len, int H, int G, int hd,
+                                         const float* sinks, int chunk, float out_factor, void* out, int n_seqs, int max_q_len, int H, int G, int hd,
                                          int vd, long long q_tok, long long q_head, long long o_tok,
                                          long long o_head, float scale, float softcap, int bias_rows,
                                          int n_lookup, int window, const float* gate,
@@ -675,7 +691,7 @@ extern "C" int gfa_scored_attention_mfma(const void* q, const void* k_pages, con
     if (q_tok % 8 || q_head % 8 || o_tok % 2 || o_head % 2) return (int)hipErrorInvalidValue;
     if ((r1 == nullptr) != (r2 == nullptr)) return (int)hipErrorInvalidValue;
     SAShape s{H, G, hd, vd, q_tok, q_head, o_tok, o_head, table_stride, window, scale, softcap,
-              bias_rows, n_lookup, sink ? 1 : 0, gate, gate_tok};
+              bias_rows, n_lookup, sink ? 1 : 0, sinks, chunk, out_factor, gate, gate_tok};
 #define SAM_GO(DK, DVT, MAXT, SPLIT) return sam_launch<DK, DVT, MAXT, SPLIT>(q, k_pages, v_pages, q_start, \
         start_pos, table, temperature, bias, lookup, talk, r1, r2, out, n_seqs, max_q_len, s, stream)
     // one token per sequence and no mix: the waves of a workgroup share a tile's key blocks

@@ -100,13 +100,14 @@ def scan(proj: torch.Tensor, layout: RowLayout, decay: torch.Tensor, state: torc
 
 def row_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], proj: torch.Tensor, layout: RowLayout,
                   eps: float, out_dtype: torch.dtype, groups: int = 1, gate: str = "sigmoid",
-                  gate_first: bool = False) -> torch.Tensor:
+                  gate_first: bool = False, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y[t, :] = o[t, :] / rms(o[t, :]) * weight * gate(g[t, :]) in ``out_dtype``, the root mean
     square taken over each of ``groups`` equal parts of the row (1: the whole row; the number
     of heads: every head by itself); o float32 [N, W]; ``weight`` float32 of W elements, or of
     fewer that divide W and are used again along the row (one weight shared by the heads), or
     None; the gate's pre-activations lie in proj at ``layout.g``; ``gate`` "sigmoid" or
-    "silu".  ``gate_first``: o is multiplied by the gate before its parts are normed."""
+    "silu".  ``gate_first``: o is multiplied by the gate before its parts are normed.  ``out``: where y
+    goes, which may be a view of wider rows (not with ``gate_first``)."""
     require_device(o, weight, proj)
     require_contiguous(o=o, weight=weight, proj=proj)
     n, width = o.shape
@@ -121,10 +122,16 @@ def row_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], proj: torch.T
         raise KernelError(f"row_norm_gate: output type {out_dtype}")
     if gate not in ("sigmoid", "silu"):
         raise KernelError(f"row_norm_gate: gate '{gate}': sigmoid or silu")
-    y = torch.empty((n, width), dtype=out_dtype, device=o.device)
+    if out is None:
+        y = torch.empty((n, width), dtype=out_dtype, device=o.device)
+    else:
+        y = out
+        if gate_first or tuple(y.shape) != (n, width) or y.dtype != out_dtype or y.stride(1) != 1 or not y.is_cuda:
+            raise KernelError("row_norm_gate: out has the wrong shape, type or strides")
     lib = library("decayed_memory")
+    stride = () if gate_first else (ctypes.c_longlong(y.stride(0)),)
     check((lib.gfa_gate_row_norm if gate_first else lib.gfa_row_norm_gate)(
         ptr(o), ptr(weight), _i(0 if weight is None else weight.numel()), ptr(proj), _i(layout.width),
-        _i(layout.g), ptr(y), _i(int(out_dtype == torch.bfloat16)), _i(n), _i(width), _i(groups),
+        _i(layout.g), ptr(y), *stride, _i(int(out_dtype == torch.bfloat16)), _i(n), _i(width), _i(groups),
         _i(int(gate == "silu")), _f(eps), stream_handle()), "row_norm_gate")
     return y

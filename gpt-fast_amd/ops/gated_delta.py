@@ -3,6 +3,7 @@ causal convolutions (ops/short_conv.py), token by token and a chunk of tokens at
 checks on the host, then the launch."""
 import ctypes
 from dataclasses import dataclass
+from typing import Optional
 
 import torch
 
@@ -17,12 +18,16 @@ MAX_KEY_DIM = 512            # rows of S a workgroup's threads hold in registers
 class RowLayout:
     """Where a token's values lie in a row of the fused projection (column offsets, in
     elements): the convolved channels q, k, v first (``conv`` of them), then the
-    pre-activations of beta and of the decay (one per head each), then the output gate."""
+    pre-activations of beta and of the decay (one per head each), then the output gate.  Where
+    the decay or the gate is a product of two matrices, ``a`` or ``g`` is the place of the first
+    one's ``a_rank`` or ``g_rank`` sums, padded to a multiple of eight."""
     width: int
     conv: int
     b: int
     a: int
     g: int
+    a_rank: int = 0
+    g_rank: int = 0
 
     @staticmethod
     def fused(n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int) -> "RowLayout":
@@ -31,6 +36,26 @@ class RowLayout:
         a = b + n_heads
         g = a + n_heads
         return RowLayout(g + n_heads * value_dim, conv, b, a, g)
+
+    @staticmethod
+    def low_rank(n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int, a_rank: int,
+                 g_rank: int) -> "RowLayout":
+        """Decay and gate (each: a rank, or 0 for none) through two matrices; every part behind the
+        convolved channels starts at a multiple of eight, and the two first products lie side by
+        side at the row's end."""
+        up = lambda n: (n + 7) // 8 * 8
+        conv = 2 * n_kv_heads * key_dim + n_heads * value_dim
+        b = up(conv)
+        a = b + n_heads                            # one per head,
+        g = up(a + (0 if a_rank else n_heads))     # or a gate as wide as the values
+        first = up(g + (0 if g_rank else n_heads * value_dim))
+        return RowLayout(first + up(a_rank) + up(g_rank), conv, b, first if a_rank else a,
+                         first + up(a_rank) if g_rank else g, up(a_rank), up(g_rank))
+
+    def shifted(self, column: int, width: int) -> "RowLayout":
+        """The same row as part of a wider one, from ``column`` on (``conv`` stays a count)."""
+        return RowLayout(width, self.conv, self.b + column, self.a + column, self.g + column, self.a_rank,
+                         self.g_rank)
 
 
 def state_size(n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int, taps: int) -> int:
@@ -61,34 +86,40 @@ def chunks_available(key_dim: int, value_dim: int) -> bool:
 
 
 def cell(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, max_q_len, n_heads,
-         n_kv_heads, key_dim, value_dim, q_scale, unit_eps) -> torch.Tensor:
+         n_kv_heads, key_dim, value_dim, q_scale, unit_eps, decays=None) -> torch.Tensor:
     """Which kernel runs the cell: token by token for short runs (single-token steps), a chunk
     of tokens at a time where some sequence brings many."""
-    chunked = max_q_len >= CHUNKS_FROM_TOKENS and chunks_available(key_dim, value_dim)
+    chunked = max_q_len >= CHUNKS_FROM_TOKENS and decays is None and chunks_available(key_dim, value_dim)
     return scan(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, n_heads, n_kv_heads,
-                key_dim, value_dim, q_scale, unit_eps, chunked=chunked, max_q_len=max_q_len)
+                key_dim, value_dim, q_scale, unit_eps, chunked=chunked, max_q_len=max_q_len, decays=decays)
 
 
 def scan(conv: torch.Tensor, proj: torch.Tensor, layout: RowLayout, A_log: torch.Tensor,
          dt_bias: torch.Tensor, state: torch.Tensor, q_start, slots, n_seqs: int, n_heads: int,
          n_kv_heads: int, key_dim: int, value_dim: int, q_scale: float, unit_eps: float,
-         chunked: bool = False, max_q_len: int = 64) -> torch.Tensor:
+         chunked: bool = False, max_q_len: int = 64, decays: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The cell over every sequence's new tokens in order; ``state`` [slots, size] holds S
     [H, dk, dv] at its start and is read and left updated.  conv float32 [N, C]: q, k, v after
     their convolutions; proj float32 [N, layout.width] holds the pre-activations of beta and
     of the decay; A_log, dt_bias float32 [H].  Returns o float32 [N, H * dv].  ``chunked``:
     the kernel that takes a chunk of tokens at a time (the same arithmetic written out; chunks
-    of 64 tokens if ``max_q_len``, the longest run of new tokens, is beyond 32, else of 32)."""
-    require_device(conv, proj, A_log, dt_bias, state, q_start, slots)
+    of 64 tokens if ``max_q_len``, the longest run of new tokens, is beyond 32, else of 32).
+    ``decays`` float32 [N, >= H * dk] (unit stride along a row): a decay per head and key channel
+    with these pre-activations; dt_bias is then float32 [H * dk]."""
+    require_device(conv, proj, A_log, dt_bias, state, q_start, slots, decays)
     require_contiguous(conv=conv, proj=proj, A_log=A_log, dt_bias=dt_bias, state=state,
                        q_start=q_start, slots=slots)
+    if decays is not None and (decays.dtype != torch.float32 or decays.dim() != 2 or decays.stride(1) != 1
+                               or decays.shape[0] != proj.shape[0] or decays.shape[1] < n_heads * key_dim):
+        raise KernelError(f"gated delta: decays must be float32 [N, >= {n_heads * key_dim}]")
     _check_step(proj, layout, state, q_start, slots, n_seqs)
     C = 2 * n_kv_heads * key_dim + n_heads * value_dim
     if conv.dtype != torch.float32 or tuple(conv.shape) != (proj.shape[0], C) or layout.conv != C:
         raise KernelError(f"gated delta: the convolved rows must be float32 [N, {C}]")
-    for name, t in (("A_log", A_log), ("dt_bias", dt_bias)):
-        if t.dtype != torch.float32 or t.numel() != n_heads:
-            raise KernelError(f"gated delta: {name} must be float32 [{n_heads}]")
+    for name, t, count in (("A_log", A_log, n_heads),
+                           ("dt_bias", dt_bias, n_heads * (1 if decays is None else key_dim))):
+        if t.dtype != torch.float32 or t.numel() != count:
+            raise KernelError(f"gated delta: {name} must be float32 [{count}]")
     if n_heads % n_kv_heads or key_dim > MAX_KEY_DIM:
         raise KernelError(f"gated delta: {n_heads} heads over {n_kv_heads} key heads of {key_dim}")
     if state.dim() != 2 or state.shape[1] < n_heads * key_dim * value_dim:
@@ -97,8 +128,11 @@ def scan(conv: torch.Tensor, proj: torch.Tensor, layout: RowLayout, A_log: torch
     lib = library("gated_delta")
     if chunked and not chunks_available(key_dim, value_dim):
         raise KernelError("gated delta: the chunked kernel does not take these sizes")
-    head = (ptr(conv), _i(C), ptr(proj), _i(layout.width), _i(layout.b), _i(layout.a), ptr(A_log),
-            ptr(dt_bias), ptr(state), _sz(state.stride(0)), ptr(q_start), ptr(slots), ptr(out), _i(n_seqs))
+    head = (ptr(conv), _i(C), ptr(proj), _i(layout.width), _i(layout.b), _i(layout.a))
+    if not chunked:
+        head += (ptr(decays), _i(0 if decays is None else decays.stride(0)))
+    head += (ptr(A_log), ptr(dt_bias), ptr(state), _sz(state.stride(0)), ptr(q_start), ptr(slots), ptr(out),
+             _i(n_seqs))
     tail = (_i(n_heads), _i(n_kv_heads), _i(key_dim), _i(value_dim), _f(q_scale), _f(unit_eps),
             stream_handle())
     if chunked:

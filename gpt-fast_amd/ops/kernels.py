@@ -107,6 +107,21 @@ def cast_rows(x: torch.Tensor, out_dtype: torch.dtype, rows: Optional[torch.Tens
 
 
 # ----------------------------------------------------------------------------- norm
+def cast_columns(x: torch.Tensor, column: int, width: int, out_dtype: torch.dtype):
+    """[N, width] in ``out_dtype``: the columns from ``column`` on of float32 rows x [N, W]."""
+    require_device(x)
+    _want(x, torch.float32, "x")
+    if x.dim() != 2 or x.stride(1) != 1 or column < 0 or column + width > x.shape[1]:
+        raise KernelError(f"cast_columns: columns {column}..{column + width - 1} of rows {tuple(x.shape)}")
+    if out_dtype not in (torch.float32, torch.bfloat16):
+        raise KernelError("cast_columns: float32 or bfloat16")
+    out = torch.empty((x.shape[0], width), dtype=out_dtype, device=x.device)
+    check(library("core").gfa_cast_columns(ptr(x[:, column:]), ctypes.c_longlong(x.stride(0)), ptr(out),
+                                           _i(x.shape[0]), _i(width), _i(int(out_dtype == torch.bfloat16)),
+                                           stream_handle()), "cast_columns")
+    return out
+
+
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
             rows: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None):
     """out[i] = x[r] * rsqrt(mean(x[r]^2) + eps) * weight, r = rows[i] if rows else i.
@@ -285,12 +300,21 @@ def attention_generic(q: torch.Tensor, k_pages, v_pages, tok_seq, tok_pos, table
 
 
 # ----------------------------------------------------------------------------- elementwise
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "clamped_swish": 2}
 
 
-def gate_mul(gu: torch.Tensor, activation: str = "silu", out: Optional[torch.Tensor] = None):
+def check_gate_limit(activation: str, limit: Optional[float]) -> float:
+    """The number the gate kernels take as their limit: only "clamped_swish" has one."""
+    if (activation == "clamped_swish") != (limit is not None):
+        raise KernelError("gate activation 'clamped_swish', and no other, takes a limit")
+    return 0.0 if limit is None else float(limit)
+
+
+def gate_mul(gu: torch.Tensor, activation: str = "silu", out: Optional[torch.Tensor] = None,
+             limit: Optional[float] = None):
     """out[n, i] = act(gu[n, i]) * gu[n, I + i]; gu [N, 2I]; act "silu" or "gelu_tanh"
-    (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))))."""
+    (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))); "clamped_swish" with ``limit``: with a =
+    min(gu[n, i], limit) and b = gu[n, I + i] clamped to -limit .. limit, ``a sigmoid(1.702 a) (b + 1)``."""
     require_device(gu)
     require_contiguous(gu=gu)
     if activation not in GATE_ACTIVATIONS:
@@ -301,14 +325,15 @@ def gate_mul(gu: torch.Tensor, activation: str = "silu", out: Optional[torch.Ten
     if out is None:
         out = torch.empty((n, two_i // 2), dtype=gu.dtype, device=gu.device)
     check(library("core").gfa_gate_mul(ptr(gu), ptr(out), _i(n), _i(two_i // 2),
-                                       _i(GATE_ACTIVATIONS[activation]), _i(_is_bf16(gu)),
+                                       _i(GATE_ACTIVATIONS[activation]),
+                                       _f(check_gate_limit(activation, limit)), _i(_is_bf16(gu)),
                                        stream_handle()), "gate_mul")
     return out
 
 
-def gate_mul_sums(gu: torch.Tensor, activation: str = "silu"):
-    """bfloat16 [N, I]: act(gu[n, i]) * gu[n, I + i] from the float32 sums gu [N, 2I] of a
-    product whose rows are the gate rows and then the up rows; one rounding."""
+def gate_mul_sums(gu: torch.Tensor, activation: str = "silu", limit: Optional[float] = None):
+    """bfloat16 [N, I]: :func:`gate_mul` of the float32 sums gu [N, 2I] of a product whose rows are
+    the gate rows and then the up rows; one rounding."""
     require_device(gu)
     require_contiguous(gu=gu)
     _want(gu, torch.float32, "gu")
@@ -319,7 +344,8 @@ def gate_mul_sums(gu: torch.Tensor, activation: str = "silu"):
         raise KernelError("gate_mul_sums: the row width must be even")
     out = torch.empty((n, two_i // 2), dtype=torch.bfloat16, device=gu.device)
     check(library("core").gfa_gate_mul_sums(ptr(gu), ptr(out), _i(n), _i(two_i // 2),
-                                            _i(GATE_ACTIVATIONS[activation]), stream_handle()),
+                                            _i(GATE_ACTIVATIONS[activation]),
+                                            _f(check_gate_limit(activation, limit)), stream_handle()),
           "gate_mul_sums")
     return out
 
@@ -449,13 +475,17 @@ def gated_normed_add(residual: torch.Tensor, y: torch.Tensor, weight: torch.Tens
 
 
 def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
-               rows: Optional[torch.Tensor] = None):
-    """out[i] = (x[r] - mean) * rsqrt(mean((x[r] - mean)^2) + eps) * weight, r = rows[i] if rows
-    else i: the layer norm with a weight and no bias.  x float32 [N, D]; weight float32 [D]."""
-    require_device(x, weight, rows)
-    require_contiguous(x=x, weight=weight, rows=rows)
+               rows: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None):
+    """out[i] = (x[r] - mean) * rsqrt(mean((x[r] - mean)^2) + eps) * weight (+ bias), r = rows[i] if
+    rows else i: the layer norm.  x float32 [N, D]; weight and bias float32 [D]."""
+    require_device(x, weight, rows, bias)
+    require_contiguous(x=x, weight=weight, rows=rows, bias=bias)
     _want(x, torch.float32, "x")
     _want(weight, torch.float32, "norm weight")
+    if bias is not None:
+        _want(bias, torch.float32, "norm bias")
+        if bias.numel() != weight.numel():
+            raise KernelError("layer_norm: weight and bias differ in size")
     if x.dim() != 2 or weight.numel() != x.shape[1]:
         raise KernelError(f"layer_norm: weight has {weight.numel()} elements, x is {tuple(x.shape)}")
     if rows is not None:
@@ -464,7 +494,7 @@ def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: tor
         raise KernelError("layer_norm: float32 or bfloat16")
     n = x.shape[0] if rows is None else rows.numel()
     out = torch.empty((n, x.shape[1]), dtype=out_dtype, device=x.device)
-    check(library("core").gfa_layer_norm(ptr(x), ptr(weight), ptr(rows), ptr(out),
+    check(library("core").gfa_layer_norm(ptr(x), ptr(weight), ptr(bias), ptr(rows), ptr(out),
                                          _i(int(out_dtype == torch.bfloat16)), _i(n), _i(x.shape[1]),
                                          _f(eps), stream_handle()), "layer_norm")
     return out

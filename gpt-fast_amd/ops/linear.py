@@ -279,12 +279,19 @@ def _linear_into(x, w, residual):
 GATE_ACTIVATIONS = K.GATE_ACTIVATIONS
 
 
-def gated_linear(x: torch.Tensor, w13: torch.Tensor, activation: str = "silu"):
+def gated_linear(x: torch.Tensor, w13: torch.Tensor, activation: str = "silu",
+                 limit: Optional[float] = None):
     """[M, I] = act(x W1^T) * (x W3^T), with w13 = rows of W1 then rows of W3
-    (model.py:227).  The few-row kernels apply either activation in their epilogue; with more
-    rows only silu has such kernels, and gelu runs the product, then the gate kernel."""
+    (model.py:227).  The few-row kernels apply silu or gelu in their epilogue; with more
+    rows only silu has such kernels, and gelu runs the product, then the gate kernel.  The clamped
+    gate (``limit``, see ``ops.kernels.gate_mul``) is always a kernel behind the product, over its
+    float32 sums where those are what the product stores."""
     if activation not in GATE_ACTIVATIONS:
         raise KernelError(f"gate activation '{activation}': {sorted(GATE_ACTIVATIONS)}")
+    if activation == "clamped_swish":
+        if x.dtype == torch.bfloat16 and x.shape[0] <= SKINNY_MAX_ROWS:
+            return K.gate_mul_sums(linear(x, w13, out_dtype=torch.float32), activation, limit)
+        return K.gate_mul(linear(x, w13), activation, limit=limit)
     if isinstance(x, HalfNormed):
         return _fast().skinny_after_chain_gated(x.xg, x.ssq, x.eps, w13, activation=activation)
     if x.dtype == torch.float32:
@@ -304,16 +311,17 @@ def gated_linear(x: torch.Tensor, w13: torch.Tensor, activation: str = "silu"):
 
 
 def gated_into(x, w13: torch.Tensor, w2: torch.Tensor, residual: torch.Tensor, then_norm=None,
-               takes_halves: bool = False, activation: str = "silu"):
+               takes_halves: bool = False, activation: str = "silu", limit: Optional[float] = None):
     """residual += (act(x W1^T) * (x W3^T)) W2^T: :func:`gated_linear`, then
     :func:`linear_into` with its arguments and result.  Between two few-row kernels that take
     and leave a norm in halves, the gate's result stays in the order the second one loads it
     in (``gemm_bf16.ChunkedRows``)."""
-    if isinstance(x, HalfNormed) and _chains(x.shape[0], x.dtype, w2, then_norm, takes_halves):
+    if isinstance(x, HalfNormed) and activation != "clamped_swish" \
+            and _chains(x.shape[0], x.dtype, w2, then_norm, takes_halves):
         h = _fast().skinny_after_chain_gated(x.xg, x.ssq, x.eps, w13, chunked=True,
                                              activation=activation)
     else:
-        h = gated_linear(x, w13, activation)
+        h = gated_linear(x, w13, activation, limit)
     return linear_into(h, w2, residual, then_norm, takes_halves)
 
 

@@ -5,11 +5,12 @@ from typing import Optional
 
 import torch
 
-from .kernels import ACTIVATIONS
+from .kernels import ACTIVATIONS, check_gate_limit
 from .library import KernelError, check, library, ptr, require_contiguous, require_device, stream_handle
 
 _i, _f, _ll = ctypes.c_int, ctypes.c_float, ctypes.c_longlong
 EXPERT_ACTIVATIONS = ("silu", "gelu_tanh", "gelu")
+CLAMPED_GATE = "clamped_swish"          # of gated experts only: ops.kernels.gate_mul
 MAX_EXPERTS = 1024
 MAX_TOP = 64
 # steps of up to this many tokens take the form of grouped_rows in which every wave reads its
@@ -79,14 +80,17 @@ def _check_experts(x, w_up, w_down, chosen, weights, gated=False):
 
 def experts_few_rows(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, chosen: torch.Tensor,
                      weights: torch.Tensor, activation: str, out: Optional[torch.Tensor] = None,
-                     gated: bool = False):
+                     gated: bool = False, limit: Optional[float] = None):
     """float32 [N, D] (+)= sum_k weights[n, k] W_down[e] act(W_up[e] x_n), e = chosen[n, k]: one
     (token, expert) pair at a time, each weight row read once per pair.  ``gated``: W_up is
     [E, 2 F, D], an expert's F gate rows and then its F up rows, and the inner row is
-    act(W_gate[e] x) * (W_up[e] x).  ``out``: the sums are added to it."""
+    act(W_gate[e] x) * (W_up[e] x), or the clamped gate with its ``limit``.  A chosen index beyond
+    the stacked experts is an identity expert: x_n itself.  ``out``: the sums are added to it."""
     _check_experts(x, w_up, w_down, chosen, weights, gated)
-    if activation not in EXPERT_ACTIVATIONS:
-        raise KernelError(f"experts: activation '{activation}': {EXPERT_ACTIVATIONS}")
+    clamped = activation == CLAMPED_GATE
+    check_gate_limit(activation, limit)
+    if (clamped and not gated) or (not clamped and activation not in EXPERT_ACTIVATIONS):
+        raise KernelError(f"experts: activation '{activation}': {EXPERT_ACTIVATIONS}, gated also {CLAMPED_GATE}")
     n, D = x.shape
     F, top = w_down.shape[2], chosen.shape[1]
     if n * top > 65535 or D * 4 > 65536 or top * F * 4 > 65536:
@@ -99,8 +103,9 @@ def experts_few_rows(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, 
     h = torch.empty((n * top, F), dtype=x.dtype, device=x.device)
     check(library("routed_experts").gfa_experts_few_rows(
         ptr(x), ptr(w_up), ptr(w_down), ptr(chosen), ptr(weights), ptr(h), ptr(out), _i(n), _i(top),
-        _i(D), _i(F), _i(ACTIVATIONS[activation]), _i(int(bool(gated))), _i(int(accumulate)),
-        _i(_is_bf16(x)), stream_handle()), "experts_few_rows")
+        _i(D), _i(F), _i(w_up.shape[0]), _i(0 if clamped else ACTIVATIONS[activation]),
+        _i(2 if clamped else int(bool(gated))), _f(limit or 0.0), _i(int(accumulate)), _i(_is_bf16(x)),
+        stream_handle()), "experts_few_rows")
     return out
 
 
@@ -136,10 +141,10 @@ def gather_pairs(x: torch.Tensor, order: torch.Tensor, top: int) -> torch.Tensor
 def gather_pairs_padded(x: torch.Tensor, order: torch.Tensor, offsets: torch.Tensor, top: int,
                         n_experts: int, cap: int) -> torch.Tensor:
     """[E, cap, D]: expert e's rows ``x[order[offsets[e] + i] // top]`` for i below its count,
-    zero rows beyond; ``cap`` must be at least the largest count (the caller's to know)."""
+    zero rows beyond (the first ``n_experts`` of the offsets' experts); ``cap`` must be at least the largest count (the caller's to know)."""
     require_device(x, order, offsets)
     require_contiguous(x=x, order=order, offsets=offsets)
-    if offsets.dtype != torch.int32 or offsets.numel() != n_experts + 1 or order.dtype != torch.int32 \
+    if offsets.dtype != torch.int32 or offsets.numel() < n_experts + 1 or order.dtype != torch.int32 \
             or cap < 1 or x.dim() != 2:
         raise KernelError("gather_pairs_padded: offsets int32 [E + 1], order int32, cap >= 1")
     out = torch.empty((n_experts, cap, x.shape[1]), dtype=x.dtype, device=x.device)
@@ -164,21 +169,29 @@ def padded_places(place: torch.Tensor, chosen: torch.Tensor, offsets: torch.Tens
 
 
 def combine_pairs(ys: torch.Tensor, place: torch.Tensor, weights: torch.Tensor,
-                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  out: Optional[torch.Tensor] = None, identity=None) -> torch.Tensor:
     """float32 [N, D] (+)= sum_k weights[n, k] ys[place[n top + k]], in the order of k; every
-    place must be a row of ys (the caller's to know)."""
-    require_device(ys, place, weights, out)
-    require_contiguous(ys=ys, place=place, weights=weights, out=out)
+    place must be a row of ys (the caller's to know).  ``identity`` = (chosen int32 [N, top],
+    number of experts, x [N, D]): a pair whose expert's index is that number or more adds
+    ``weights[n, k] x[n]`` instead, and its place is not looked at."""
+    chosen, n_experts, x = identity if identity is not None else (None, 0, None)
+    require_device(ys, place, weights, out, chosen, x)
+    require_contiguous(ys=ys, place=place, weights=weights, out=out, chosen=chosen, x=x)
     n, top = weights.shape
     D = ys.shape[1]
-    if ys.shape[0] < n * top or place.numel() != n * top or weights.dtype != torch.float32:
+    if (ys.shape[0] < n * top and identity is None) or place.numel() != n * top or weights.dtype != torch.float32:
         raise KernelError("combine_pairs: ys [>= N top, D], place [N top] and weights [N, top] do not fit")
+    if identity is not None and (chosen.dtype != torch.int32 or chosen.numel() != n * top
+                                 or tuple(x.shape) != (n, D)):
+        raise KernelError("combine_pairs: identity needs chosen int32 [N, top] and x [N, D]")
     accumulate = out is not None
     if out is None:
         out = torch.empty((n, D), dtype=torch.float32, device=ys.device)
     elif tuple(out.shape) != (n, D) or out.dtype != torch.float32:
         raise KernelError("combine_pairs: out must be float32 [N, D]")
-    check(library("routed_experts").gfa_combine_pairs(ptr(ys), ptr(place), ptr(weights), ptr(out), _i(n),
+    check(library("routed_experts").gfa_combine_pairs(ptr(ys), ptr(place), ptr(weights), ptr(chosen),
+                                                      _i(n_experts), ptr(x),
+                                                      _i(0 if x is None else _is_bf16(x)), ptr(out), _i(n),
                                                       _i(top), _i(D), _i(int(accumulate)),
                                                       _i(_is_bf16(ys)), stream_handle()), "combine_pairs")
     return out
@@ -205,8 +218,8 @@ def grouped_rows(x: torch.Tensor, order: Optional[torch.Tensor], top: int, w: to
     if not grouped_rows_take(x, w):
         raise KernelError("grouped_rows: bfloat16 x [rows, K] and W [E, N, K] with K a multiple of 8")
     E, N, K = w.shape
-    if offsets.dtype != torch.int32 or offsets.numel() != E + 1:
-        raise KernelError(f"grouped_rows: offsets must be int32 [{E + 1}]")
+    if offsets.dtype != torch.int32 or offsets.numel() < E + 1:
+        raise KernelError(f"grouped_rows: offsets must be int32 [>= {E + 1}]")
     if order is not None:
         if order.dtype != torch.int32 or top < 1 or order.numel() > x.shape[0] * top:
             raise KernelError("grouped_rows: order must be int32 with at most rows * top elements")

@@ -52,14 +52,17 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
               scale: float, *, window: int = 0, temperature: Optional[torch.Tensor] = None,
               softcap: float = 0.0, bias: Optional[torch.Tensor] = None,
               lookup: Optional[torch.Tensor] = None, talk: Optional[torch.Tensor] = None,
-              log_bias=None, sink: bool = False, gate: Optional[torch.Tensor] = None,
+              log_bias=None, sink: bool = False, sinks: Optional[torch.Tensor] = None, chunk: int = 0,
+              out_factor: float = 1.0, gate: Optional[torch.Tensor] = None,
               head_major: bool = False, out: Optional[torch.Tensor] = None, step=None) -> torch.Tensor:
     """Each token's heads attend to the keys of its sequence's pages.  q is [N, H, hd], or
     [H, N, hd] if ``head_major`` (the result then lies the same way); k_pages
     [pages, G, 64, hd], v_pages [pages, G, vd, 64]; temperature float32 [H]; bias float32
     [rows, H] with lookup int32 [distances] (see :func:`distance_rows`); talk float32 [H, H];
     log_bias = (r1, r2), float32 [H] each: ``r1[h] ln(1 + r2[h] (i - j))`` is taken off the
-    score; sink: the softmax's denominator has one more term exp(0); gate float32 [N, >= H], a
+    score; sink: the softmax's denominator has one more term exp(0), or with ``sinks`` float32 [H]
+    exp(sinks[h]); chunk: only keys of the query's own chunk of so many positions (0: all);
+    ``out_factor``: the result is multiplied by it before it is rounded; gate float32 [N, >= H], a
     view of wider rows allowed: head h of token n is multiplied by ``sigmoid(gate[n, h])``.
     Returns [N, H, vd] (or [H, N, vd]) in q's type.  ``out`` may be a view with unit stride
     in its last dimension.  ``step`` = (q_start int32 [B + 1], start_pos int32 [B], B, longest
@@ -67,9 +70,11 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
     of sizes the matrix-core kernel takes go there."""
     r1, r2 = log_bias if log_bias is not None else (None, None)
     require_device(q, k_pages, v_pages, tok_seq, tok_pos, table, temperature, bias, lookup, talk, out,
-                   r1, r2, gate)
+                   r1, r2, gate, sinks)
     require_contiguous(tok_seq=tok_seq, tok_pos=tok_pos, table=table, temperature=temperature,
-                       bias=bias, lookup=lookup, talk=talk, r1=r1, r2=r2)
+                       bias=bias, lookup=lookup, talk=talk, r1=r1, r2=r2, sinks=sinks)
+    if chunk < 0 or (sinks is not None and not sink):
+        raise KernelError("scored attention: chunk must be 0 or a size, and sinks go with sink")
     if q.dim() != 3 or q.stride(2) != 1:
         raise KernelError("scored attention: q must have three dimensions, the last with unit stride")
     n, H = (q.shape[1], q.shape[0]) if head_major else (q.shape[0], q.shape[1])
@@ -86,7 +91,7 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
     if (r1 is None) != (r2 is None):
         raise KernelError("scored attention: the bias by log distance needs both r1 and r2")
     for name, t, count in (("temperature", temperature, H), ("talk", talk, H * H), ("r1", r1, H),
-                           ("r2", r2, H)):
+                           ("r2", r2, H), ("sinks", sinks, H)):
         if t is not None and (t.dtype != torch.float32 or t.numel() != count):
             raise KernelError(f"scored attention: {name} must be float32 with {count} elements")
     if gate is not None and (gate.dtype != torch.float32 or gate.dim() != 2 or gate.shape[0] != n
@@ -124,7 +129,7 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
         check(lib.gfa_scored_attention_mfma(
             ptr(q), ptr(k_pages), ptr(v_pages), ptr(q_start), ptr(start_pos), ptr(table),
             _i(table.shape[1]), ptr(temperature), ptr(bias), ptr(lookup if bias is not None else None),
-            ptr(talk), ptr(r1), ptr(r2), _i(int(sink)), ptr(out), _i(n_seqs), _i(max_q_len), _i(H),
+            ptr(talk), ptr(r1), ptr(r2), _i(int(sink)), ptr(sinks), _i(chunk), _f(out_factor), ptr(out), _i(n_seqs), _i(max_q_len), _i(H),
             _i(G), _i(hd), _i(vd),
             _ll(q.stride(tok)), _ll(q.stride(head)), _ll(out.stride(tok)), _ll(out.stride(head)),
             _f(scale), _f(softcap or 0.0), _i(rows), _i(0 if lookup is None else lookup.numel()),
@@ -133,7 +138,7 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tok
     check(lib.gfa_scored_attention(
         ptr(q), ptr(k_pages), ptr(v_pages), ptr(tok_seq), ptr(tok_pos), ptr(table),
         _i(table.shape[1]), ptr(temperature), ptr(bias), ptr(lookup if bias is not None else None),
-        ptr(talk), ptr(r1), ptr(r2), _i(int(sink)), ptr(out), _i(n), _i(H), _i(G), _i(hd), _i(vd),
+        ptr(talk), ptr(r1), ptr(r2), _i(int(sink)), ptr(sinks), _i(chunk), _f(out_factor), ptr(out), _i(n), _i(H), _i(G), _i(hd), _i(vd),
         _ll(q.stride(tok)),
         _ll(q.stride(head)), _ll(out.stride(tok)), _ll(out.stride(head)), _f(scale),
         _f(softcap or 0.0), _i(rows), _i(0 if lookup is None else lookup.numel()), _i(window or 0),
@@ -155,11 +160,11 @@ def unit_heads_store(proj: torch.Tensor, bias: Optional[torch.Tensor], tok_seq, 
     pairs (i, i + rotary_dim / 2)) with cos and sin times ``trig_scale``; keys and values put
     into the cache (k_pages None: not)."""
     require_device(proj, bias, tok_seq, tok_pos, table, k_pages, v_pages, q_weight, k_weight, freqs)
-    require_contiguous(proj=proj, bias=bias, tok_seq=tok_seq, tok_pos=tok_pos, table=table,
+    require_contiguous(bias=bias, tok_seq=tok_seq, tok_pos=tok_pos, table=table,
                        q_weight=q_weight, k_weight=k_weight, freqs=freqs)
     width = (n_heads + n_kv_heads) * head_dim + n_kv_heads * value_dim
-    if proj.dtype != torch.float32 or proj.dim() != 2 or proj.shape[1] < width:
-        raise KernelError(f"unit_heads_store: proj must be float32 [N, >= {width}]")
+    if proj.dtype != torch.float32 or proj.dim() != 2 or proj.shape[1] < width or proj.stride(1) != 1:
+        raise KernelError(f"unit_heads_store: proj must be float32 [N, >= {width}], a view of wider rows is allowed")
     if bias is not None and (bias.dtype != torch.float32 or bias.numel() != width):
         raise KernelError(f"unit_heads_store: bias must be float32 [{width}]")
     for name, t in (("q_weight", q_weight), ("k_weight", k_weight)):
@@ -177,7 +182,7 @@ def unit_heads_store(proj: torch.Tensor, bias: Optional[torch.Tensor], tok_seq, 
         raise KernelError("unit_heads_store: token maps are shorter than the batch")
     q = torch.empty((n, n_heads, head_dim), dtype=out_dtype, device=proj.device)
     check(library("scored_attention").gfa_unit_heads_store(
-        ptr(proj), _i(proj.shape[1]), ptr(bias), ptr(q), ptr(k_pages), ptr(v_pages), ptr(tok_seq),
+        ptr(proj), _i(proj.stride(0)), ptr(bias), ptr(q), ptr(k_pages), ptr(v_pages), ptr(tok_seq),
         ptr(tok_pos), ptr(table), _i(table.shape[1]), _i(n), _i(n_heads), _i(n_kv_heads),
         _i(head_dim), _i(value_dim), _f(-1.0 if eps is None else eps), ptr(q_weight), ptr(k_weight),
         ptr(freqs if rotary_dim else None), _i(rotary_dim), _i(layout), _f(trig_scale),

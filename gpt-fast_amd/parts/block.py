@@ -5,6 +5,7 @@ from ..config.spec import LayerSpec
 from ..ops import kernels as K
 from ..ops import linear as L
 from ..ops import streams as ST
+from ..ops import term_join as TJ
 from .base import (FEED_FORWARDS, MIXERS, NORMS, Param, Part, ResidualStream, Runtime, check_bound,
                    register_block)
 
@@ -303,8 +304,9 @@ class PostNormBlock(PreNormBlock):
         if spec.feed_forward is not None:
             self.feed_forward_out_norm = NORMS.build(spec.feed_forward_out_norm, runtime)
         for norm in (self.mixer_out_norm, self.feed_forward_out_norm):
-            if norm is not None and not hasattr(norm, "layer_form"):
-                raise TypeError("a post_norm block's sums take a norm with layer_form() (kind 'layer')")
+            if norm is not None and (not hasattr(norm, "layer_form") or norm.spec.bias):
+                raise TypeError("a post_norm block's sums take a norm with layer_form() (kind 'layer') and "
+                                "without a bias")
         self.alpha = float(spec.residual_scale)
         self.mixer_scale = self.feed_forward_scale = None
         if spec.layer_scale:
@@ -329,7 +331,7 @@ class PostNormBlock(PreNormBlock):
         the new stream, from the same kernel where that is the rows themselves, else by the
         norm's own kernel; None without a next norm.  ``result`` is a tensor or a
         ``(first, second, (w_first, w_second), eps)`` of two branches."""
-        weight, eps = out_norm.layer_form()
+        weight, _, eps = out_norm.layer_form()
         ls = scale.weight if scale is not None else None
         plain = next_norm is not None and getattr(next_norm, "plain_rows", False)
         args = dict(alpha=self.alpha, layer_scale=ls, out_dtype=self.rt.dtype if plain else None)
@@ -480,7 +482,82 @@ class HyperConnectedBlock(PreNormBlock):
             stream.tensor                    # a caller with a plain tensor gets the sums now
 
 
+class ParallelBlock(PreNormBlock):
+    """``x <- x + m (mixer(h) + ffn(h))`` with ``h = norm(x)``, one norm (the spec's ``mixer_norm``) for
+    both and m its ``result_scale``; without a feed-forward the mixer alone.  Both sublayers hand
+    over their results, and one kernel adds them to the stream and makes the rows of the norm that
+    reads it next (a layer norm, an RMS norm or none); it is therefore put off until the stream is
+    read next.  What a sublayer can offer, best first: ``forward_terms(x, batch[, entry]) ->
+    [(rows, factor)]``; ``forward_last -> (operand, matrix)`` of its last product, which the block
+    then runs in whatever form is fastest (partial sums are added on the kernel's way);
+    ``forward_rows``; plain ``forward``."""
+
+    takes_stream = True
+    takes_prepared = False
+    libraries = ("term_join",)
+
+    def __init__(self, spec: LayerSpec, runtime: Runtime):
+        if spec.feed_forward_norm is not None:
+            raise ValueError("a parallel block has one norm, its mixer_norm")
+        self.spec = spec
+        self.rt = runtime
+        self.mixer_norm = NORMS.build(spec.mixer_norm, runtime)
+        self.mixer = MIXERS.build(spec.mixer, runtime)
+        self.feed_forward_norm = self.feed_forward = None
+        if spec.feed_forward is not None:
+            self.feed_forward = FEED_FORWARDS.build(spec.feed_forward, runtime)
+        self.factor = float(spec.result_scale)
+
+    def children(self):
+        s = self.spec
+        out = {s.mixer_norm_name: self.mixer_norm, s.mixer_name: self.mixer}
+        if self.feed_forward is not None:
+            out[s.feed_forward_name] = self.feed_forward
+        return out
+
+    def _terms(self, part, args, like):
+        """[(rows, factor)] of a sublayer."""
+        if hasattr(part, "forward_terms"):
+            return [(y, f * self.factor) for y, f in part.forward_terms(*args)]
+        if hasattr(part, "forward_last"):
+            return [(L.linear_terms(*part.forward_last(*args)), self.factor)]
+        if hasattr(part, "forward_rows"):
+            return [(part.forward_rows(*args), self.factor)]
+        y = torch.zeros_like(like)
+        part.forward(*args, y)
+        return [(y, self.factor)]
+
+    def _join(self, residual, terms, next_norm):
+        """The terms into the stream; the rows of ``next_norm`` over it, or None."""
+        while len(terms) > TJ.MAX_TERMS:
+            TJ.join(residual, terms[:TJ.MAX_TERMS])
+            terms = terms[TJ.MAX_TERMS:]
+        kind, weight, bias, eps = None, None, None, 0.0
+        if getattr(next_norm, "plain_rows", False):
+            kind = "plain"
+        elif hasattr(next_norm, "layer_form"):
+            kind, (weight, bias, eps) = "layer", next_norm.layer_form()
+        elif hasattr(next_norm, "row_and_column_form"):
+            kind, (weight, eps) = "rms", next_norm.row_and_column_form()
+        out = TJ.join(residual, terms, kind, weight, bias, eps, self.rt.dtype if kind else None)
+        if next_norm is None or kind:
+            return out
+        return next_norm.forward(residual)
+
+    def forward(self, residual, batch, entry):
+        stream = residual if isinstance(residual, ResidualStream) else ResidualStream(residual)
+        x = stream.normed(self.mixer_norm)
+        like = stream.tensor
+        terms = self._terms(self.mixer, (x, batch, entry), like)
+        if self.feed_forward is not None:
+            terms = terms + self._terms(self.feed_forward, (x, batch), like)
+        stream.defer(lambda rows, then_norm, halves: self._join(rows, terms, then_norm))
+        if stream is not residual:
+            stream.tensor                    # a caller with a plain tensor gets the sums now
+
+
 register_block("pre_norm", PreNormBlock)
+register_block("parallel", ParallelBlock)
 register_block("hyper_connected", HyperConnectedBlock)
 register_block("post_norm", PostNormBlock)
 register_block("sandwich_norm", SandwichNormBlock)

@@ -10,13 +10,15 @@ from .base import Param, Part, Runtime, add_late, check_bound, register_feed_for
 
 
 class GatedFeedForward(Part):
-    """``w2( act(w1 x) * (w3 x) )`` without biases, act = silu or the tanh form of gelu.  w1
+    """``w2( act(w1 x) * (w3 x) )`` without biases, act = silu, the tanh form of gelu or the clamped
+    gate (``ops.kernels.gate_mul``).  w1
     and w3 are one matrix ``w13`` (rows of w1, then rows of w3) so that the gate is applied
     where the products end."""
 
     def __init__(self, spec: GatedFeedForwardSpec, runtime: Runtime):
         if spec.activation not in L.GATE_ACTIVATIONS:
             raise ValueError(f"activation '{spec.activation}': {sorted(L.GATE_ACTIVATIONS)}")
+        K.check_gate_limit(spec.activation, spec.limit)
         self.spec = spec
         self.rt = runtime
         self.w13 = self.w2 = None
@@ -43,7 +45,11 @@ class GatedFeedForward(Part):
         # both products wait until the stream is read next: whether the gate's result stays in
         # the order the second product loads it in depends on the norm that follows
         add_late(residual, lambda rows, then_norm, takes_halves: L.gated_into(
-            x, self.w13, self.w2, rows, then_norm, takes_halves, self.spec.activation))
+            x, self.w13, self.w2, rows, then_norm, takes_halves, self.spec.activation, self.spec.limit))
+
+    def forward_last(self, x, batch):
+        """The operand and the matrix of the last product, which the block runs."""
+        return L.gated_linear(x, self.w13, self.spec.activation, self.spec.limit), self.w2
 
 
 register_feed_forward("gated", GatedFeedForward)

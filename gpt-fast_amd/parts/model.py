@@ -77,7 +77,9 @@ class DecoderModel:
         extra = sorted(set(tensors) - set(declared))
         if extra:
             raise KeyError(f"model: parameters {extra} belong to no part")
-        self._tensors = dict(tensors)
+        # (place, elements, bytes per element) of every parameter; the tensors themselves belong to
+        # the parts, which may keep them in another form
+        self._sizes = {name: (t.data_ptr(), t.numel(), t.element_size()) for name, t in tensors.items()}
         self.embedding = tensors[self.plan.embedding_name]
         self.head = tensors[self.plan.head_name]
         prefix = self.plan.final_norm_name + "."
@@ -105,14 +107,9 @@ class DecoderModel:
             parts = list(self.blocks) + list(self.input_adds) + [self.input_position]
             unread = sum(getattr(p, "unread_bytes", lambda r: 0)(rows) for p in parts if p is not None)
             return self.parameter_bytes(exclude_embedding) - unread
-        seen, total = set(), 0
-        for name, t in self._tensors.items():
-            if exclude_embedding and name == self.plan.embedding_name \
-                    and t.data_ptr() != self.head.data_ptr():
-                continue
-            if t.data_ptr() not in seen:
-                seen.add(t.data_ptr())
-                total += t.numel() * t.element_size()
+        total = 0
+        for n, size in self._read_once(exclude_embedding):
+            total += n * size
         return total
 
     @property
@@ -129,15 +126,18 @@ class DecoderModel:
     def parameter_count(self, exclude_embedding: bool = True) -> int:
         """Elements of the same parameters (the reference's ``params`` of
         generate.py:251-268, which feeds its FLOPS line)."""
-        seen, total = set(), 0
-        for name, t in self._tensors.items():
-            if exclude_embedding and name == self.plan.embedding_name \
-                    and t.data_ptr() != self.head.data_ptr():
+        return sum(n for n, _ in self._read_once(exclude_embedding))
+
+    def _read_once(self, exclude_embedding: bool):
+        """(elements, bytes per element) of every parameter a step reads, shared ones once."""
+        head = self._sizes[self.plan.head_name][0]
+        seen = set()
+        for name, (place, n, size) in self._sizes.items():
+            if exclude_embedding and name == self.plan.embedding_name and place != head:
                 continue
-            if t.data_ptr() not in seen:
-                seen.add(t.data_ptr())
-                total += t.numel()
-        return total
+            if place not in seen:
+                seen.add(place)
+                yield n, size
 
     # ------------------------------------------------------------------ cache
     def cache_needs(self) -> List[object]:

@@ -71,30 +71,36 @@ class NoNorm(Part):
 
 
 class LayerNorm(Part):
-    """``(x - mean) * rsqrt(mean((x - mean)^2) + eps) * weight`` over the last dimension, no
-    bias; statistics in float32 from the float32 stream, one rounding to the compute type at
-    the store.  ``layer_form()`` tells a kernel that completes the stream how to apply it on
-    its way."""
+    """``(x - mean) * rsqrt(mean((x - mean)^2) + eps) * weight`` over the last dimension, plus a
+    bias per element if the spec has one; statistics in float32 from the float32 stream, one
+    rounding to the compute type at the store.  ``layer_form()`` tells a kernel that completes the
+    stream how to apply it on its way."""
 
     replayable = True
 
     def __init__(self, spec: NormSpec, runtime: Runtime):
         self.spec = spec
         self.rt = runtime
-        self.weight = None
+        self.weight = self.bias = None
 
     def parameters(self):
-        return {"weight": Param((self.spec.dim,), role="vector", init="norm")}
+        p = {"weight": Param((self.spec.dim,), role="vector", init="norm")}
+        if self.spec.bias:
+            p["bias"] = Param((self.spec.dim,), role="vector", init="around_zero")
+        return p
 
     def bind(self, tensors):
         check_bound("LayerNorm", self.parameters(), tensors)
         self.weight = tensors["weight"].to(torch.float32).contiguous()
+        if self.spec.bias:
+            self.bias = tensors["bias"].to(torch.float32).contiguous()
 
     def forward(self, residual: torch.Tensor, rows=None) -> torch.Tensor:
-        return K.layer_norm(residual, self.weight, self.spec.eps, self.rt.dtype, rows=rows)
+        return K.layer_norm(residual, self.weight, self.spec.eps, self.rt.dtype, rows=rows, bias=self.bias)
 
     def layer_form(self):
-        return self.weight, self.spec.eps
+        """(weight, bias or None, eps)."""
+        return self.weight, self.bias, self.spec.eps
 
 
 register_norm("rms", RMSNorm)

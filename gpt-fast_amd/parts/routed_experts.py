@@ -30,7 +30,8 @@ class RoutedExperts(Part):
     weights are worked out in float32 by one kernel per step.  The experts' matrices are
     stacked, ``w_up [E, F, D]`` (gated: ``[E, 2 F, D]``, an expert's gate rows and then its up
     rows) and ``w_down [E, D, F]``.  The shared expert has the same form; with ``shared_gate``
-    its result is multiplied by ``sigmoid(w_sg x)``, one number per token.
+    its result is multiplied by ``sigmoid(w_sg x)``, one number per token.  ``identity`` further
+    router outputs stand behind the experts': their expert is x itself.
 
     Few rows (and every single-token step, so that a recorded step never asks the host): in
     bfloat16 the pairs are put in the order of their experts on the device and one kernel per
@@ -47,12 +48,21 @@ class RoutedExperts(Part):
     replayable = True          # single-token steps read nothing on the host
 
     def __init__(self, spec: RoutedExpertsSpec, runtime: Runtime):
-        if spec.activation not in RE.EXPERT_ACTIVATIONS:
-            raise ValueError(f"activation '{spec.activation}': {RE.EXPERT_ACTIVATIONS}")
-        if spec.n_experts % spec.n_groups or not 1 <= spec.keep_groups <= spec.n_groups or \
-                not 1 <= spec.top <= spec.keep_groups * (spec.n_experts // spec.n_groups):
-            raise ValueError(f"routed experts: top {spec.top} of {spec.n_experts} experts in "
+        clamped = spec.activation == RE.CLAMPED_GATE
+        if spec.activation not in RE.EXPERT_ACTIVATIONS and not (clamped and spec.gated):
+            raise ValueError(f"activation '{spec.activation}': {RE.EXPERT_ACTIVATIONS}, gated also {RE.CLAMPED_GATE}")
+        if spec.identity < 0:
+            raise ValueError(f"routed experts: {spec.identity} identity experts")
+        # what the router, the correction and the choice cover
+        self.n_choices = spec.n_experts + spec.identity
+        if self.n_choices % spec.n_groups or not 1 <= spec.keep_groups <= spec.n_groups or \
+                not 1 <= spec.top <= spec.keep_groups * (self.n_choices // spec.n_groups):
+            raise ValueError(f"routed experts: top {spec.top} of {self.n_choices} experts in "
                              f"{spec.n_groups} groups of which {spec.keep_groups} are kept")
+        if (spec.limit is not None) != clamped or \
+                (spec.shared_limit is not None) != (clamped and spec.shared_hidden > 0):
+            raise ValueError(f"routed experts: limits go with {RE.CLAMPED_GATE}, one for the experts and one "
+                             f"for a shared expert")
         self.spec = spec
         self.rt = runtime
         if spec.scoring not in RE.ROUTER_SCORINGS or not 1 <= spec.group_top <= RE.MAX_GROUP_TOP:
@@ -67,11 +77,11 @@ class RoutedExperts(Part):
 
     def parameters(self):
         s = self.spec
-        p = {"w_router": Param((s.n_experts, s.dim)),
+        p = {"w_router": Param((self.n_choices, s.dim)),
              "w_up": Param((s.n_experts, self.up_rows, s.dim)),
              "w_down": Param((s.n_experts, s.dim, s.hidden))}
         if s.choice_correction:
-            p["correction"] = Param((s.n_experts,), role="vector", init="around_zero")
+            p["correction"] = Param((self.n_choices,), role="vector", init="around_zero")
         if s.shared_hidden:
             p["shared_up"] = Param(((2 if s.gated else 1) * s.shared_hidden, s.dim))
             p["shared_down"] = Param((s.dim, s.shared_hidden))
@@ -95,7 +105,7 @@ class RoutedExperts(Part):
     def step_flops(self, q_lens, starts) -> float:
         s = self.spec
         mats = 3 if s.gated else 2
-        per_token = s.n_experts * s.dim + mats * s.top * s.hidden * s.dim + mats * s.shared_hidden * s.dim
+        per_token = self.n_choices * s.dim + mats * s.top * s.hidden * s.dim + mats * s.shared_hidden * s.dim
         return 2.0 * sum(q_lens) * per_token
 
     def unread_bytes(self, rows: int) -> int:
@@ -105,33 +115,35 @@ class RoutedExperts(Part):
         s = self.spec
         last = self.last_chosen
         if last is not None and last.shape[0] == rows:
-            idle = s.n_experts - int(torch.unique(last).numel())
+            named = torch.unique(last)
+            idle = s.n_experts - int((named < s.n_experts).sum())
         else:
-            idle = int(s.n_experts * (1.0 - s.top / s.n_experts) ** rows)
+            idle = int(s.n_experts * (1.0 - s.top / self.n_choices) ** rows)
         per_expert = (self.w_up[0].numel() + self.w_down[0].numel()) * self.w_up.element_size()
         return idle * per_expert
 
     def _routed(self, x, chosen, weights, y, batch):
         s = self.spec
         n = x.shape[0]
+        identity = (chosen, s.n_experts, x) if s.identity else None
         few = n <= PAIRWISE_MAX_ROWS or getattr(batch, "is_decode", False)
         if few and n >= GROUPED_MIN_ROWS and RE.grouped_rows_take(x, self.w_up) and s.hidden % 8 == 0:
-            offsets, order, place = RE.expert_order(chosen, s.n_experts)
+            offsets, order, place = RE.expert_order(chosen, self.n_choices)
             if s.gated:
                 # the float32 sums of the gate rows and the up rows, then the gate
                 sums = RE.grouped_rows(x, order, s.top, self.w_up, offsets, None, n)
-                h = K.gate_mul_sums(sums, s.activation)
+                h = K.gate_mul_sums(sums, s.activation, s.limit)
             else:
                 h = RE.grouped_rows(x, order, s.top, self.w_up, offsets, s.activation, n)
             ys = RE.grouped_rows(h, None, 1, self.w_down, offsets, None, n)
-            return RE.combine_pairs(ys, place, weights, out=y)
+            return RE.combine_pairs(ys, place, weights, out=y, identity=identity)
         if few:
             return RE.experts_few_rows(x, self.w_up, self.w_down, chosen, weights, s.activation, out=y,
-                                       gated=s.gated)
-        offsets, order, place = RE.expert_order(chosen, s.n_experts)
+                                       gated=s.gated, limit=s.limit)
+        offsets, order, place = RE.expert_order(chosen, self.n_choices)
         bounds = offsets.cpu().tolist()                         # the host learns the experts' shares
         most = max(bounds[e + 1] - bounds[e] for e in range(s.n_experts))
-        cap = (most + PAD_ROWS_TO - 1) // PAD_ROWS_TO * PAD_ROWS_TO
+        cap = max(1, (most + PAD_ROWS_TO - 1) // PAD_ROWS_TO) * PAD_ROWS_TO
         if s.n_experts * cap <= PADDED_MAX_WASTE * n * s.top:
             # shares of similar size: each padded to the largest, one batched product for all
             xs = RE.gather_pairs_padded(x, order, offsets, s.top, s.n_experts, cap)
@@ -141,8 +153,9 @@ class RoutedExperts(Part):
             ys = torch.empty((s.n_experts, cap, s.dim), dtype=x.dtype, device=x.device)
             self._batched(hs, self.w_down, ys)
             return RE.combine_pairs(ys.view(-1, s.dim), RE.padded_places(place, chosen, offsets, cap),
-                                    weights, out=y)
-        xs = RE.gather_pairs(x, order, s.top)
+                                    weights, out=y, identity=identity)
+        # (the pairs of identity experts stand behind the others and take part in no product)
+        xs = RE.gather_pairs(x, order[:bounds[s.n_experts]], s.top)
         hs = torch.empty((xs.shape[0], self.up_rows), dtype=x.dtype, device=x.device)
         ys = torch.empty((xs.shape[0], s.dim), dtype=x.dtype, device=x.device)
         for e in range(s.n_experts):
@@ -154,12 +167,12 @@ class RoutedExperts(Part):
             a, b = bounds[e], bounds[e + 1]
             if b > a:
                 self._product(hs[a:b], self.w_down[e], ys[a:b])
-        return RE.combine_pairs(ys, place, weights, out=y)
+        return RE.combine_pairs(ys, place, weights, out=y, identity=identity)
 
     def _activated(self, h):
         """The inner rows from the first product's rows [P, F] (or [P, 2 F]: gate, then up)."""
         if self.spec.gated:
-            return K.gate_mul(h, self.spec.activation)
+            return K.gate_mul(h, self.spec.activation, limit=self.spec.limit)
         return K.activate(h, self.spec.activation, out=h)
 
     def _batched(self, a, w, out):
@@ -177,19 +190,19 @@ class RoutedExperts(Part):
         """The feed-forward's output alone, float32 [N, D]."""
         s = self.spec
         z = L.linear(x, self.w_router, out_dtype=torch.float32)
-        chosen, weights = RE.route(z, s.n_experts, s.top, s.n_groups, s.keep_groups, s.weight_eps,
+        chosen, weights = RE.route(z, self.n_choices, s.top, s.n_groups, s.keep_groups, s.weight_eps,
                                    scoring=s.scoring, correction=self.correction, group_top=s.group_top)
         self.last_chosen = chosen                  # a replayed step leaves its choice here as well
         y = None
         if s.shared_hidden:
             if s.gated:
-                h = L.gated_linear(x, self.shared_up, s.activation)
+                h = L.gated_linear(x, self.shared_up, s.activation, s.shared_limit)
             else:
                 h = L.linear(x, self.shared_up)
                 K.activate(h, s.activation, out=h)
             y = L.linear(h, self.shared_down, out_dtype=torch.float32)
             if self.shared_gate:
-                K.scale_rows_sigmoid(y, z[:, s.n_experts:])
+                K.scale_rows_sigmoid(y, z[:, self.n_choices:])
         return self._routed(x, chosen, weights, y, batch)
 
     def forward(self, x, batch, residual):
