@@ -19,7 +19,7 @@ import time
 HERE = os.path.dirname(os.path.abspath(__file__))
 MODULES = ("core", "sampling", "gemm_bf16", "gemm_wide_bf16", "gemm_tiled_bf16", "attention_bf16",
            "matrix_memory", "differential_attention", "decayed_memory", "scored_attention", "latent_attention",
-           "routed_experts", "gated_delta", "short_conv", "state_space", "streams", "term_join",
+           "routed_experts", "gated_delta", "delta_chunks", "short_conv", "state_space", "streams", "term_join",
            "ceilings")
 ARCH = "gfx950"
 FLAGS = ["-O3", "-std=c++17", "-fPIC", "-shared", f"--offload-arch={ARCH}",

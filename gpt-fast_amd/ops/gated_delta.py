@@ -1,6 +1,7 @@
-"""Python faces of the gated-delta-rule kernels of csrc/gated_delta.hip: the cell behind the short
-causal convolutions (ops/short_conv.py), token by token and a chunk of tokens at a time.  Shape
-checks on the host, then the launch."""
+"""Python faces of the gated-delta-rule kernels of csrc/gated_delta.hip and csrc/delta_chunks.hip: the
+cell behind the short causal convolutions (ops/short_conv.py), token by token, a chunk of tokens at
+a time in one kernel, and all chunks at once with one small kernel that walks them.  Shape checks on
+the host, then the launch."""
 import ctypes
 from dataclasses import dataclass
 from typing import Optional
@@ -85,11 +86,27 @@ def chunks_available(key_dim: int, value_dim: int) -> bool:
     return bool(library("gated_delta").gfa_gated_delta_chunks_take(_i(key_dim), _i(value_dim)))
 
 
+PARALLEL_CHUNK = 64          # tokens per chunk of csrc/delta_chunks.hip
+# (sequence, chunk, head) triples whose intermediate matrices are in memory at once (0.2 MB each for
+# 128 x 128 heads); longer prompts go through in several rounds
+PARALLEL_TRIPLES = 8192
+
+
+def parallel_chunks_available(key_dim: int, value_dim: int) -> bool:
+    return bool(library("delta_chunks").gfa_delta_chunks_take(_i(key_dim), _i(value_dim)))
+
+
 def cell(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, max_q_len, n_heads,
          n_kv_heads, key_dim, value_dim, q_scale, unit_eps, decays=None) -> torch.Tensor:
-    """Which kernel runs the cell: token by token for short runs (single-token steps), a chunk
-    of tokens at a time where some sequence brings many."""
-    chunked = max_q_len >= CHUNKS_FROM_TOKENS and decays is None and chunks_available(key_dim, value_dim)
+    """Which kernels run the cell: token by token for short runs (single-token steps), chunks of
+    tokens where some sequence brings many."""
+    chunked = False
+    if max_q_len >= CHUNKS_FROM_TOKENS:
+        if parallel_chunks_available(key_dim, value_dim):
+            return parallel_chunks(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs,
+                                   max_q_len, n_heads, n_kv_heads, key_dim, value_dim, q_scale, unit_eps,
+                                   decays=decays)
+        chunked = decays is None and chunks_available(key_dim, value_dim)
     return scan(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, n_heads, n_kv_heads,
                 key_dim, value_dim, q_scale, unit_eps, chunked=chunked, max_q_len=max_q_len, decays=decays)
 
@@ -106,6 +123,61 @@ def scan(conv: torch.Tensor, proj: torch.Tensor, layout: RowLayout, A_log: torch
     of 64 tokens if ``max_q_len``, the longest run of new tokens, is beyond 32, else of 32).
     ``decays`` float32 [N, >= H * dk] (unit stride along a row): a decay per head and key channel
     with these pre-activations; dt_bias is then float32 [H * dk]."""
+    C, out = _check_cell(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, n_heads, n_kv_heads,
+                         key_dim, value_dim, decays)
+    lib = library("gated_delta")
+    if chunked and (decays is not None or not chunks_available(key_dim, value_dim)):
+        raise KernelError("gated delta: the chunked kernel does not take these sizes")
+    head = (ptr(conv), _i(C), ptr(proj), _i(layout.width), _i(layout.b), _i(layout.a))
+    if not chunked:
+        head += (ptr(decays), _i(0 if decays is None else decays.stride(0)))
+    head += (ptr(A_log), ptr(dt_bias), ptr(state), _sz(state.stride(0)), ptr(q_start), ptr(slots), ptr(out),
+             _i(n_seqs))
+    tail = (_i(n_heads), _i(n_kv_heads), _i(key_dim), _i(value_dim), _f(q_scale), _f(unit_eps),
+            stream_handle())
+    if chunked:
+        check(lib.gfa_gated_delta_chunks(*head, _i(int(max_q_len)), *tail), "gated_delta_chunks")
+    else:
+        check(lib.gfa_gated_delta_scan(*head, *tail), "gated_delta_scan")
+    return out
+
+
+def parallel_chunks(conv, proj, layout: RowLayout, A_log, dt_bias, state, q_start, slots, n_seqs: int,
+                    max_q_len: int, n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int,
+                    q_scale: float, unit_eps: float, decays: Optional[torch.Tensor] = None,
+                    chunks_at_once: Optional[int] = None) -> torch.Tensor:
+    """:func:`scan` over chunks of 64 tokens: what a chunk does to the state, whatever the state is,
+    is worked out for all chunks at once, and a small kernel walks them (csrc/delta_chunks.hip).
+    ``max_q_len``: the longest run of new tokens; ``chunks_at_once``: chunks of each sequence per
+    round (None: by PARALLEL_TRIPLES)."""
+    C, out = _check_cell(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, n_heads, n_kv_heads,
+                         key_dim, value_dim, decays)
+    if not parallel_chunks_available(key_dim, value_dim):
+        raise KernelError("gated delta: the parallel chunks' kernels do not take these sizes")
+    lib = library("delta_chunks")
+    chunks = (int(max_q_len) + PARALLEL_CHUNK - 1) // PARALLEL_CHUNK
+    seg = chunks_at_once or max(1, PARALLEL_TRIPLES // (n_seqs * n_heads))
+    seg = min(seg, chunks)
+    sizes = [ctypes.c_int() for _ in range(4)]
+    lib.gfa_delta_chunks_floats(_i(key_dim), _i(value_dim), *(ctypes.byref(n) for n in sizes))
+    triples = n_seqs * seg * n_heads
+    room = torch.empty(triples * sum(n.value for n in sizes), dtype=torch.float32, device=proj.device)
+    parts, at = [], 0
+    for n in sizes:                                # every size is a multiple of 256 floats
+        parts.append(room[at:])
+        at += triples * n.value
+    check(lib.gfa_delta_chunks(
+        ptr(conv), _i(C), ptr(proj), _i(layout.width), _i(layout.b), _i(layout.a), ptr(decays),
+        _i(0 if decays is None else decays.stride(0)), ptr(A_log), ptr(dt_bias), ptr(state),
+        _sz(state.stride(0)), ptr(q_start), ptr(slots), ptr(out), *(ptr(p) for p in parts), _i(n_seqs),
+        _i(int(max_q_len)), _i(seg), _i(n_heads), _i(n_kv_heads), _i(key_dim), _i(value_dim), _f(q_scale),
+        _f(unit_eps), stream_handle()), "delta_chunks")
+    return out
+
+
+def _check_cell(conv, proj, layout, A_log, dt_bias, state, q_start, slots, n_seqs, n_heads, n_kv_heads, key_dim,
+                value_dim, decays):
+    """Shape checks of the cell's arguments: (convolved channels, a new tensor for the result)."""
     require_device(conv, proj, A_log, dt_bias, state, q_start, slots, decays)
     require_contiguous(conv=conv, proj=proj, A_log=A_log, dt_bias=dt_bias, state=state,
                        q_start=q_start, slots=slots)
@@ -125,18 +197,4 @@ def scan(conv: torch.Tensor, proj: torch.Tensor, layout: RowLayout, A_log: torch
     if state.dim() != 2 or state.shape[1] < n_heads * key_dim * value_dim:
         raise KernelError("gated delta: the state is smaller than S [H, dk, dv]")
     out = torch.empty((proj.shape[0], n_heads * value_dim), dtype=torch.float32, device=proj.device)
-    lib = library("gated_delta")
-    if chunked and not chunks_available(key_dim, value_dim):
-        raise KernelError("gated delta: the chunked kernel does not take these sizes")
-    head = (ptr(conv), _i(C), ptr(proj), _i(layout.width), _i(layout.b), _i(layout.a))
-    if not chunked:
-        head += (ptr(decays), _i(0 if decays is None else decays.stride(0)))
-    head += (ptr(A_log), ptr(dt_bias), ptr(state), _sz(state.stride(0)), ptr(q_start), ptr(slots), ptr(out),
-             _i(n_seqs))
-    tail = (_i(n_heads), _i(n_kv_heads), _i(key_dim), _i(value_dim), _f(q_scale), _f(unit_eps),
-            stream_handle())
-    if chunked:
-        check(lib.gfa_gated_delta_chunks(*head, _i(int(max_q_len)), *tail), "gated_delta_chunks")
-    else:
-        check(lib.gfa_gated_delta_scan(*head, *tail), "gated_delta_scan")
-    return out
+    return C, out

@@ -34,7 +34,7 @@ class GatedDelta(Part):
     both second matrices (zeros between them) takes their sums to the channels."""
 
     replayable = True
-    libraries = ("gated_delta", "short_conv", "decayed_memory")
+    libraries = ("gated_delta", "delta_chunks", "short_conv", "decayed_memory")
     defers_sum = True              # ``residual`` may be a parts.base.ResidualStream
 
     def __init__(self, spec: GatedDeltaSpec, runtime: Runtime):
