@@ -684,3 +684,192 @@ extern "C" int gfa_grouped_rows(const void* x, const int* order, int top, const 
 #undef GFA_LAUNCH_GROUPED
     return GFA_LAUNCH_RESULT();
 }
+
+// --------------------------------------------------------------------------------------
+// Prompts in bfloat16: the experts' products over the pairs in the order of their experts, all
+// experts in one launch and nothing read on the host.
+//
+//   out[p, n] = f(W[e][n, :] . x[row(p), :])   for the pairs p of every expert e
+//
+// row(p) = order[p] / top if order is given, else p.  Rows are cut into tiles of 128 that do not cross
+// experts; expert_tiles_kernel lists them as (expert, first row), -1 behind the last.  A workgroup
+// makes a 128 x 128 tile, its four waves 64 x 64 each, K in pieces of 64 that are fetched a piece
+// ahead and go through two buffers of shared memory whose 16-byte chunks are swizzled by the row.
+// The products are formed transposed (A = W, B = x), so that a lane holds four columns of one row.
+// Gated experts (W_up [2 F, D]: gate rows, then up rows): every second 16-column tile of a workgroup is
+// of the up rows, so a wave holds both halves of its pairs, and the gate is applied to the float sums.
+// The workgroups of one XCD (every eighth) take consecutive row tiles of the same columns: those of
+// one expert meet its matrix in that XCD's cache.
+#define ET_ROWS 128
+#define ET_COLS 128
+#define ET_K 64
+
+__global__ __launch_bounds__(1024) void expert_tiles_kernel(const int* __restrict__ offsets, int E,
+                                                            int* __restrict__ tiles, int n_tiles) {
+    extern __shared__ int et_start[];                  // [E + 1]
+    if (threadIdx.x == 0) {
+        int at = 0;
+        for (int e = 0; e < E; ++e) {
+            et_start[e] = at;
+            at += (offsets[e + 1] - offsets[e] + ET_ROWS - 1) / ET_ROWS;
+        }
+        et_start[E] = at;
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e < E; e += blockDim.x)
+        for (int i = et_start[e]; i < et_start[e + 1] && i < n_tiles; ++i) {
+            tiles[2 * i] = e;
+            tiles[2 * i + 1] = offsets[e] + (i - et_start[e]) * ET_ROWS;
+        }
+    for (int i = et_start[E] + threadIdx.x; i < n_tiles; i += blockDim.x) tiles[2 * i] = -1;
+}
+
+extern "C" int gfa_expert_tiles(const int* offsets, int E, int* tiles, int n_tiles, hipStream_t stream) {
+    if (n_tiles <= 0) return 0;
+    if (E <= 0 || E > 8192) return (int)hipErrorInvalidValue;
+    expert_tiles_kernel<<<1, 1024, sizeof(int) * (size_t)(E + 1), stream>>>(offsets, E, tiles, n_tiles);
+    return GFA_LAUNCH_RESULT();
+}
+
+// mode 0: the sums; 1: act(sum); 2: act(gate) * up; 3: the clamped gate.  F: columns of out (modes 2, 3:
+// W has 2 F rows).
+template <bool GATED>
+__global__ __launch_bounds__(256) void expert_tile_kernel(
+        const bf16_t* __restrict__ x, const int* __restrict__ order, int top, const bf16_t* __restrict__ w,
+        const int* __restrict__ offsets, const int* __restrict__ tiles, int n_tiles, int n_cols,
+        bf16_t* __restrict__ out, int F, int K, int mode, int act, float limit) {
+    __shared__ __attribute__((aligned(16))) char et_lds[2][(ET_ROWS + ET_COLS) * ET_K * 2];
+    const int total = n_tiles * n_cols, per = (total + 7) / 8;
+    const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if (work >= total) return;                         // the whole workgroup
+    const int mt = work % n_tiles, nt = work / n_tiles;
+    const int e = tiles[2 * mt];
+    if (e < 0) return;
+    const int m0 = tiles[2 * mt + 1], m1 = offsets[e + 1];
+    const int N = GATED ? 2 * F : F;
+    const bf16_t* we = w + (size_t)e * N * K;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int li = lane & 15, lg = lane >> 4;
+    const int wm = (wave & 1) * 64, wn = (wave >> 1) * 64;
+    // this thread's 16-byte chunks of a piece: rows r0 + 32 i of x and of W, chunk c of their eight.
+    // Rows and columns beyond the tile's read the last one again and are never stored; beyond K the
+    // chunks of W are zero.
+    const int r0 = tid >> 3, c = tid & 7;
+    const bf16_t *x0, *x1, *x2, *x3, *w0, *w1, *w2, *w3;
+    {
+        auto x_row = [&](int r) {
+            const int m = m0 + r < m1 ? m0 + r : m1 - 1;
+            return x + (size_t)(order ? order[m] / top : m) * K + c * 8;
+        };
+        auto w_row = [&](int r) {
+            int n;
+            if (GATED) {
+                const int t = r >> 4;                  // even tiles: gate rows, odd: the same up rows
+                n = nt * (ET_COLS / 2) + (t >> 1) * 16 + (r & 15);
+                n = (n < F ? n : F - 1) + ((t & 1) ? F : 0);
+            } else {
+                n = nt * ET_COLS + r;
+                n = n < F ? n : F - 1;
+            }
+            return we + (size_t)n * K + c * 8;
+        };
+        x0 = x_row(r0); x1 = x_row(r0 + 32); x2 = x_row(r0 + 64); x3 = x_row(r0 + 96);
+        w0 = w_row(r0); w1 = w_row(r0 + 32); w2 = w_row(r0 + 64); w3 = w_row(r0 + 96);
+    }
+    uint4 xr0, xr1, xr2, xr3, wr0, wr1, wr2, wr3;
+#define ET_FETCH(k) do { \
+        const int kc = (k) + c * 8 < K ? (k) : -c * 8;             /* beyond K: the row's first chunk */ \
+        xr0 = *(const uint4*)(x0 + kc); xr1 = *(const uint4*)(x1 + kc); \
+        xr2 = *(const uint4*)(x2 + kc); xr3 = *(const uint4*)(x3 + kc); \
+        wr0 = *(const uint4*)(w0 + kc); wr1 = *(const uint4*)(w1 + kc); \
+        wr2 = *(const uint4*)(w2 + kc); wr3 = *(const uint4*)(w3 + kc); \
+        if ((k) + c * 8 >= K) wr0 = wr1 = wr2 = wr3 = make_uint4(0, 0, 0, 0); \
+    } while (0)
+    re_floatx4_t acc[4][4];                            // [column tile][row tile]
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = re_floatx4_t{0.f, 0.f, 0.f, 0.f};
+    ET_FETCH(0);
+    int buf = 0;
+    const int put = r0 * (ET_K * 2) + ((c ^ (r0 & 7)) << 4);       // (r0 + 32 i) & 7 is r0 & 7
+    for (int k0 = 0; k0 < K; k0 += ET_K, buf ^= 1) {
+        char* X = et_lds[buf];
+        char* W = X + ET_ROWS * ET_K * 2;
+        *(uint4*)(X + put) = xr0;
+        *(uint4*)(X + put + 32 * ET_K * 2) = xr1;
+        *(uint4*)(X + put + 64 * ET_K * 2) = xr2;
+        *(uint4*)(X + put + 96 * ET_K * 2) = xr3;
+        *(uint4*)(W + put) = wr0;
+        *(uint4*)(W + put + 32 * ET_K * 2) = wr1;
+        *(uint4*)(W + put + 64 * ET_K * 2) = wr2;
+        *(uint4*)(W + put + 96 * ET_K * 2) = wr3;
+        __syncthreads();
+        if (k0 + ET_K < K) ET_FETCH(k0 + ET_K);
+#pragma unroll
+        for (int kk = 0; kk < ET_K / 32; ++kk) {
+            ReFrag a[4], b[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int rn = wn + i * 16 + li, rm = wm + i * 16 + li, ch = kk * 4 + lg;
+                a[i].u = *(const uint4*)(W + rn * (ET_K * 2) + ((ch ^ (rn & 7)) << 4));
+                b[i].u = *(const uint4*)(X + rm * (ET_K * 2) + ((ch ^ (rm & 7)) << 4));
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i].v, b[j].v, acc[i][j], 0, 0, 0);
+        }
+    }
+#undef ET_FETCH
+    const bool wide = F % 4 == 0;                      // four columns at once (out starts at a multiple of 8 bytes)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int m = m0 + wm + j * 16 + li;
+        if (m >= m1) continue;
+#pragma unroll
+        for (int i = 0; i < 4; i += GATED ? 2 : 1) {
+            const int n = GATED ? nt * (ET_COLS / 2) + (wn + i * 16) / 2 + lg * 4 : nt * ET_COLS + wn + i * 16 + lg * 4;
+            bf16_t v[4];
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                float s = acc[i][j][q];
+                if (GATED) {
+                    const float u = acc[i + (GATED ? 1 : 0)][j][q];
+                    s = mode == 3 ? re_clamped_pair(s, u, limit) : re_activation(s, act) * u;
+                } else if (mode == 1) {
+                    s = re_activation(s, act);
+                }
+                v[q] = float_to_bf16(s);
+            }
+            bf16_t* dst = out + (size_t)m * F + n;
+            if (wide && n + 4 <= F) {
+                *(uint2*)dst = make_uint2((uint32_t)v[0] | ((uint32_t)v[1] << 16), (uint32_t)v[2] | ((uint32_t)v[3] << 16));
+            } else {
+#pragma unroll
+                for (int q = 0; q < 4; ++q)
+                    if (n + q < F) dst[q] = v[q];
+            }
+        }
+    }
+}
+
+extern "C" int gfa_expert_tile_product(const void* x, const int* order, int top, const void* w,
+                                       const int* offsets, const int* tiles, int n_tiles, void* out, int F,
+                                       int K, int mode, int act, float limit, hipStream_t stream) {
+    if (n_tiles <= 0) return 0;
+    if (F <= 0 || K <= 0 || K % 8 || top <= 0 || mode < 0 || mode > 3 || (act != 0 && act != 1 && act != 3))
+        return (int)hipErrorInvalidValue;
+    const int n_cols = mode >= 2 ? (F + ET_COLS / 2 - 1) / (ET_COLS / 2) : (F + ET_COLS - 1) / ET_COLS;
+    const long long total = (long long)n_tiles * n_cols;
+    if (total > 0x7ffffff0LL / 2) return (int)hipErrorInvalidValue;
+    const unsigned grid = (unsigned)((total + 7) / 8 * 8);
+    if (mode >= 2)
+        expert_tile_kernel<true><<<grid, 256, 0, stream>>>((const bf16_t*)x, order, top, (const bf16_t*)w, offsets,
+                                                           tiles, n_tiles, n_cols, (bf16_t*)out, F, K, mode, act, limit);
+    else
+        expert_tile_kernel<false><<<grid, 256, 0, stream>>>((const bf16_t*)x, order, top, (const bf16_t*)w, offsets,
+                                                            tiles, n_tiles, n_cols, (bf16_t*)out, F, K, mode, act, limit);
+    return GFA_LAUNCH_RESULT();
+}

@@ -726,8 +726,9 @@ extern "C" int gfa_scored_attention_mfma(const void* q, const void* k_pages, con
 // of every head of q and k are turned by pos * freqs[i], pairs (2i, 2i + 1) (layout 0) or
 // (i, i + rot / 2) (layout 1), with cos and sin multiplied by `trig` (rot 0: no rotation).
 // q goes to q_out [N, H, d]; keys and values to the token's place in the cache (skipped if
-// k_pages is null).  One workgroup per token, one wave per head vector, float arithmetic, one
-// rounding at the store.
+// k_pages is null).  A workgroup takes `per_block` head vectors of one token (a launch of few tokens
+// spreads them over the chip), one wave per head vector; the angles' cosines and sines are worked out
+// once per workgroup.  Float arithmetic, one rounding at the store.
 template <typename T>
 __global__ __launch_bounds__(SA_THREADS) void unit_heads_store_kernel(
         const float* __restrict__ proj, int row_width, const float* __restrict__ bias,
@@ -735,15 +736,24 @@ __global__ __launch_bounds__(SA_THREADS) void unit_heads_store_kernel(
         const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
         const int* __restrict__ table, int table_stride, int H, int G, int d, int dv, float eps,
         const float* __restrict__ wq, const float* __restrict__ wk,
-        const float* __restrict__ freqs, int rot, int layout, float trig) {
+        const float* __restrict__ freqs, int rot, int layout, float trig, int per_block) {
+    extern __shared__ float uh_turn[];                 // [rot / 2] cosines, [rot / 2] sines, times trig
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n = blockIdx.x;
     const float* row = proj + (size_t)n * row_width;
     const int pos = tok_pos[n];
+    for (int i = threadIdx.x; i < rot / 2; i += SA_THREADS) {
+        float sn, cs;
+        sincosf((float)pos * freqs[i], &sn, &cs);
+        uh_turn[i] = cs * trig;
+        uh_turn[rot / 2 + i] = sn * trig;
+    }
+    if (rot) __syncthreads();
+    const int u_end = (int)(blockIdx.y + 1) * per_block < H + 2 * G ? (int)(blockIdx.y + 1) * per_block : H + 2 * G;
     const int page = k_pages ? table[(size_t)tok_seq[n] * table_stride + pos / GFA_PAGE] : 0;
     const int slot = pos % GFA_PAGE;
     const int half = rot >> 1;
-    for (int u = wave; u < H + 2 * G; u += SA_WAVES) {
+    for (int u = blockIdx.y * per_block + wave; u < u_end; u += SA_WAVES) {
         const bool is_q = u < H, is_k = !is_q && u < H + G;
         const int width = (is_q || is_k) ? d : dv;
         const int off = is_q ? u * d : (is_k ? H * d + (u - H) * d : (H + G) * d + (u - H - G) * dv);
@@ -765,9 +775,9 @@ __global__ __launch_bounds__(SA_THREADS) void unit_heads_store_kernel(
                 const bool first = layout == 0 ? (e & 1) == 0 : e < half;
                 const int p = layout == 0 ? (e ^ 1) : (first ? e + half : e - half);
                 const float y = (row[off + p] + (bias ? bias[off + p] : 0.f)) * r * (hw ? hw[p] : 1.f);
-                float sn, cs;
-                sincosf((float)pos * freqs[layout == 0 ? e >> 1 : (first ? e : e - half)], &sn, &cs);
-                x = first ? (x * cs - y * sn) * trig : (x * cs + y * sn) * trig;
+                const int i = layout == 0 ? e >> 1 : (first ? e : e - half);
+                const float cs = uh_turn[i], sn = uh_turn[half + i];
+                x = first ? x * cs - y * sn : x * cs + y * sn;
             }
             if (is_q) store_from_float(q_out + ((size_t)n * H + u) * d + e, x);
             else if (is_k) store_from_float(k_pages + key_elem(page, u - H, slot, e, G, d), x);
@@ -785,14 +795,21 @@ extern "C" int gfa_unit_heads_store(const float* proj, int row_width, const floa
     if (n_tokens <= 0) return 0;
     if (rot < 0 || rot > d || rot % 2 || (rot && !freqs) || (layout != 0 && layout != 1))
         return (int)hipErrorInvalidValue;
+    // enough workgroups for the chip's compute units, and at most four head vectors' waves idle
+    const int units = H + 2 * G;
+    int blocks = n_tokens >= 512 ? 1 : (512 + n_tokens - 1) / n_tokens;
+    if (blocks > (units + SA_WAVES - 1) / SA_WAVES) blocks = (units + SA_WAVES - 1) / SA_WAVES;
+    const int per_block = ((units + blocks - 1) / blocks + SA_WAVES - 1) / SA_WAVES * SA_WAVES;
+    const dim3 grid(n_tokens, (units + per_block - 1) / per_block);
+    const size_t shmem = sizeof(float) * (size_t)rot;
     if (is_bf16)
-        unit_heads_store_kernel<bf16_t><<<n_tokens, SA_THREADS, 0, stream>>>(
+        unit_heads_store_kernel<bf16_t><<<grid, SA_THREADS, shmem, stream>>>(
             proj, row_width, bias, (bf16_t*)q_out, (bf16_t*)k_pages, (bf16_t*)v_pages, tok_seq,
-            tok_pos, table, table_stride, H, G, d, dv, eps, wq, wk, freqs, rot, layout, trig);
+            tok_pos, table, table_stride, H, G, d, dv, eps, wq, wk, freqs, rot, layout, trig, per_block);
     else
-        unit_heads_store_kernel<float><<<n_tokens, SA_THREADS, 0, stream>>>(
+        unit_heads_store_kernel<float><<<grid, SA_THREADS, shmem, stream>>>(
             proj, row_width, bias, (float*)q_out, (float*)k_pages, (float*)v_pages, tok_seq,
-            tok_pos, table, table_stride, H, G, d, dv, eps, wq, wk, freqs, rot, layout, trig);
+            tok_pos, table, table_stride, H, G, d, dv, eps, wq, wk, freqs, rot, layout, trig, per_block);
     return GFA_LAUNCH_RESULT();
 }
 

@@ -235,3 +235,58 @@ def grouped_rows(x: torch.Tensor, order: Optional[torch.Tensor], top: int, w: to
         _i(-1 if activation is None else ACTIVATIONS[activation]), _i(max(1, int(rows_at_most))),
         _i(int(rows_at_most <= DIRECT_X_MAX_ROWS)), stream_handle()), "grouped_rows")
     return out
+
+
+TILE_ROWS = 128              # rows of a tile of expert_tile_product (csrc/routed_experts.hip: ET_ROWS)
+
+
+def expert_tiles(offsets: torch.Tensor, n_experts: int, pairs: int) -> torch.Tensor:
+    """int32 [T, 2]: the tiles of up to 128 rows into which the experts' pairs (their places by
+    ``offsets``) fall, as (expert, first row), -1 behind the last; T is what ``pairs`` pairs can make
+    at most."""
+    require_device(offsets)
+    require_contiguous(offsets=offsets)
+    if offsets.dtype != torch.int32 or offsets.numel() < n_experts + 1:
+        raise KernelError(f"expert_tiles: offsets must be int32 [>= {n_experts + 1}]")
+    n = pairs // TILE_ROWS + min(n_experts, pairs)
+    tiles = torch.empty((n, 2), dtype=torch.int32, device=offsets.device)
+    check(library("routed_experts").gfa_expert_tiles(ptr(offsets), _i(n_experts), ptr(tiles), _i(n),
+                                                     stream_handle()), "expert_tiles")
+    return tiles
+
+
+def expert_tile_product(x: torch.Tensor, order: Optional[torch.Tensor], top: int, w: torch.Tensor,
+                        offsets: torch.Tensor, tiles: torch.Tensor, pairs: int,
+                        activation: Optional[str] = None, gated: bool = False,
+                        limit: Optional[float] = None) -> torch.Tensor:
+    """bfloat16 [pairs, F]: row p of expert e is ``act(W[e] x[r])``, r = ``order[p] // top`` (or p itself
+    without ``order``); ``gated``: W is [E, 2 F, K] and the row ``act(W_gate x) * (W_up x)``, or the
+    clamped gate.  Rows that belong to no expert of ``tiles`` are not written.  Operands as for
+    :func:`grouped_rows`; nothing is read on the host."""
+    require_device(x, order, w, offsets, tiles)
+    require_contiguous(x=x, order=order, w=w, offsets=offsets, tiles=tiles)
+    if not grouped_rows_take(x, w):
+        raise KernelError("expert_tile_product: bfloat16 x [rows, K] and W [E, N, K] with K a multiple of 8")
+    E, N, K = w.shape
+    if gated and N % 2:
+        raise KernelError("expert_tile_product: gated experts have an even number of rows")
+    if offsets.dtype != torch.int32 or offsets.numel() < E + 1 or tiles.dtype != torch.int32 or tiles.dim() != 2 \
+            or tiles.shape[1] != 2:
+        raise KernelError(f"expert_tile_product: offsets int32 [>= {E + 1}], tiles int32 [T, 2]")
+    if order is not None and (order.dtype != torch.int32 or order.numel() < pairs or pairs > x.shape[0] * top):
+        raise KernelError("expert_tile_product: order must be int32 and name every pair")
+    if order is None and pairs > x.shape[0]:
+        raise KernelError("expert_tile_product: more pairs than rows")
+    clamped = activation == CLAMPED_GATE
+    check_gate_limit(activation, limit)
+    if (clamped and not gated) or (activation is None and gated) or \
+            (activation is not None and not clamped and activation not in EXPERT_ACTIVATIONS):
+        raise KernelError(f"expert_tile_product: activation '{activation}'")
+    F = N // 2 if gated else N
+    out = torch.empty((pairs, F), dtype=torch.bfloat16, device=x.device)
+    mode = 3 if clamped else (2 if gated else (1 if activation is not None else 0))
+    check(library("routed_experts").gfa_expert_tile_product(
+        ptr(x), ptr(order), _i(max(1, top)), ptr(w), ptr(offsets), ptr(tiles), _i(tiles.shape[0]), ptr(out), _i(F),
+        _i(K), _i(mode), _i(0 if clamped or activation is None else ACTIVATIONS[activation]), _f(limit or 0.0),
+        stream_handle()), "expert_tile_product")
+    return out

@@ -14,8 +14,8 @@ PAIRWISE_MAX_ROWS = 16
 # from this many rows on, bfloat16 steps of few rows put the pairs in the order of their experts
 # on the device and read each expert's matrices once for all of its rows
 GROUPED_MIN_ROWS = 1
-# prompts: the experts' shares of the pairs are padded to the largest share (rounded up to this
-# many rows) and all experts are one batched product, unless the padded rows are more than this
+# prompts in float32: the experts' shares of the pairs are padded to the largest share (rounded up to
+# this many rows) and all experts are one batched product, unless the padded rows are more than this
 # many times the pairs (a router that sends most tokens to few experts): then one product per
 # expert over its own rows
 PAD_ROWS_TO = 32
@@ -37,12 +37,13 @@ class RoutedExperts(Part):
     bfloat16 the pairs are put in the order of their experts on the device and one kernel per
     product reads each expert's matrix once for all of its rows (matrix cores); in float32, and
     for sizes that kernel does not take, kernels that take one (token, expert) pair at a time.
-    More rows: the pairs are put in the
-    order of their experts on the device and the host reads where each expert's rows begin;
-    shares of similar size are padded to the largest and all experts are ONE batched product,
-    else each expert's rows are one product (the matrix library for bfloat16, the library's own
-    float32 kernels otherwise); a last kernel adds every token's pairs in the order of its
-    choice, so the result does not depend on what else the step holds."""
+    More rows: the pairs are put in the order of their experts on the device.  In bfloat16 one kernel
+    per product takes the experts' rows in tiles, the gate or activation in the first one's epilogue.
+    In float32 (and for sizes that kernel does not take) the host reads where each expert's rows
+    begin; shares of similar size are padded to the largest and all experts are ONE batched product
+    of the library's own kernel, else each expert's rows are one product.  A last kernel adds every
+    token's pairs in the order of its choice, so the result does not depend on what else the step
+    holds."""
 
     libraries = ("routed_experts",)
     replayable = True          # single-token steps read nothing on the host
@@ -141,17 +142,23 @@ class RoutedExperts(Part):
             return RE.experts_few_rows(x, self.w_up, self.w_down, chosen, weights, s.activation, out=y,
                                        gated=s.gated, limit=s.limit)
         offsets, order, place = RE.expert_order(chosen, self.n_choices)
+        if RE.grouped_rows_take(x, self.w_up) and s.hidden % 8 == 0:
+            tiles = RE.expert_tiles(offsets, s.n_experts, n * s.top)
+            hs = RE.expert_tile_product(x, order, s.top, self.w_up, offsets, tiles, n * s.top, s.activation,
+                                        s.gated, s.limit)
+            ys = RE.expert_tile_product(hs, None, 1, self.w_down, offsets, tiles, n * s.top)
+            return RE.combine_pairs(ys, place, weights, out=y, identity=identity)
         bounds = offsets.cpu().tolist()                         # the host learns the experts' shares
         most = max(bounds[e + 1] - bounds[e] for e in range(s.n_experts))
         cap = max(1, (most + PAD_ROWS_TO - 1) // PAD_ROWS_TO) * PAD_ROWS_TO
-        if s.n_experts * cap <= PADDED_MAX_WASTE * n * s.top:
+        if x.dtype == torch.float32 and s.n_experts * cap <= PADDED_MAX_WASTE * n * s.top:
             # shares of similar size: each padded to the largest, one batched product for all
             xs = RE.gather_pairs_padded(x, order, offsets, s.top, s.n_experts, cap)
             hs = torch.empty((s.n_experts, cap, self.up_rows), dtype=x.dtype, device=x.device)
-            self._batched(xs, self.w_up, hs)
+            K.gemm_f32_batched(xs, self.w_up, hs)
             hs = self._activated(hs.view(-1, self.up_rows)).view(s.n_experts, cap, s.hidden)
             ys = torch.empty((s.n_experts, cap, s.dim), dtype=x.dtype, device=x.device)
-            self._batched(hs, self.w_down, ys)
+            K.gemm_f32_batched(hs, self.w_down, ys)
             return RE.combine_pairs(ys.view(-1, s.dim), RE.padded_places(place, chosen, offsets, cap),
                                     weights, out=y, identity=identity)
         # (the pairs of identity experts stand behind the others and take part in no product)
@@ -174,12 +181,6 @@ class RoutedExperts(Part):
         if self.spec.gated:
             return K.gate_mul(h, self.spec.activation, limit=self.spec.limit)
         return K.activate(h, self.spec.activation, out=h)
-
-    def _batched(self, a, w, out):
-        """out[e] = a[e] w[e]^T for every expert: a [E, cap, K], w [E, M, K], out [E, cap, M]."""
-        if a.dtype == torch.float32:
-            return K.gemm_f32_batched(a, w, out)
-        return torch.bmm(a, w.transpose(1, 2), out=out)         # the vendor library, as for prompts
 
     def _product(self, a, w, out):
         if a.dtype == torch.float32:
