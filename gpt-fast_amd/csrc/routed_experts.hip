@@ -694,7 +694,8 @@ extern "C" int gfa_grouped_rows(const void* x, const int* order, int top, const 
 // row(p) = order[p] / top if order is given, else p.  Rows are cut into tiles of 128 that do not cross
 // experts; expert_tiles_kernel lists them as (expert, first row), -1 behind the last.  A workgroup
 // makes a 128 x 128 tile, its four waves 64 x 64 each, K in pieces of 64 that are fetched a piece
-// ahead and go through two buffers of shared memory whose 16-byte chunks are swizzled by the row.
+// ahead and go through shared memory, whose 16-byte chunks are swizzled by the row (one buffer: three
+// workgroups share a compute unit, which hides more than a second buffer with two did).
 // The products are formed transposed (A = W, B = x), so that a lane holds four columns of one row.
 // Gated experts (W_up [2 F, D]: gate rows, then up rows): every second 16-column tile of a workgroup is
 // of the up rows, so a wave holds both halves of its pairs, and the gate is applied to the float sums.
@@ -734,11 +735,11 @@ extern "C" int gfa_expert_tiles(const int* offsets, int E, int* tiles, int n_til
 // mode 0: the sums; 1: act(sum); 2: act(gate) * up; 3: the clamped gate.  F: columns of out (modes 2, 3:
 // W has 2 F rows).
 template <bool GATED>
-__global__ __launch_bounds__(256) void expert_tile_kernel(
+__global__ __launch_bounds__(256, 3) void expert_tile_kernel(
         const bf16_t* __restrict__ x, const int* __restrict__ order, int top, const bf16_t* __restrict__ w,
         const int* __restrict__ offsets, const int* __restrict__ tiles, int n_tiles, int n_cols,
         bf16_t* __restrict__ out, int F, int K, int mode, int act, float limit) {
-    __shared__ __attribute__((aligned(16))) char et_lds[2][(ET_ROWS + ET_COLS) * ET_K * 2];
+    __shared__ __attribute__((aligned(16))) char et_lds[(ET_ROWS + ET_COLS) * ET_K * 2];
     const int total = n_tiles * n_cols, per = (total + 7) / 8;
     const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if (work >= total) return;                         // the whole workgroup
@@ -791,11 +792,11 @@ __global__ __launch_bounds__(256) void expert_tile_kernel(
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = re_floatx4_t{0.f, 0.f, 0.f, 0.f};
     ET_FETCH(0);
-    int buf = 0;
     const int put = r0 * (ET_K * 2) + ((c ^ (r0 & 7)) << 4);       // (r0 + 32 i) & 7 is r0 & 7
-    for (int k0 = 0; k0 < K; k0 += ET_K, buf ^= 1) {
-        char* X = et_lds[buf];
+    for (int k0 = 0; k0 < K; k0 += ET_K) {
+        char* X = et_lds;
         char* W = X + ET_ROWS * ET_K * 2;
+        __syncthreads();
         *(uint4*)(X + put) = xr0;
         *(uint4*)(X + put + 32 * ET_K * 2) = xr1;
         *(uint4*)(X + put + 64 * ET_K * 2) = xr2;
