@@ -57,7 +57,8 @@ __global__ __launch_bounds__(64) void route_kernel(
     for (int e = lane; e < E; e += 64) c[e] = s[e] + (correction ? correction[e] : 0.f);
     __syncthreads();
     const int per = E / groups;
-    for (int g = lane; g < groups; g += 64) {
+    const bool choose_groups = keep < groups;           // else every group stays
+    for (int g = lane; choose_groups && g < groups; g += 64) {
         // the sum of the group's largest scores: the largest, then the largest of the rest, ...
         int taken[RE_MAX_GROUP_TOP];
         float total = 0.f;
@@ -78,7 +79,7 @@ __global__ __launch_bounds__(64) void route_kernel(
         gscore[g] = total;
     }
     __syncthreads();
-    for (int g = lane; g < groups; g += 64) {
+    for (int g = lane; choose_groups && g < groups; g += 64) {
         int better = 0;
         for (int o = 0; o < groups; ++o)
             better += (gscore[o] > gscore[g] || (gscore[o] == gscore[g] && o < g)) ? 1 : 0;
@@ -90,7 +91,7 @@ __global__ __launch_bounds__(64) void route_kernel(
 #pragma unroll
     for (int i = 0; i < RE_MAX_PER_LANE; ++i) {
         const int e = lane + 64 * i;
-        mine[i] = (e < E && allowed[e / per]) ? c[e] : -INFINITY;
+        mine[i] = (e < E && (!choose_groups || allowed[e / per])) ? c[e] : -INFINITY;
     }
     float total = 0.f;
     float w_k = 0.f;                                    // lane k keeps the k-th choice

@@ -242,6 +242,51 @@ def test_clamped_experts_and_identity_experts(dtype, tol, E, I, top, D, Fh, shar
     assert named or not I                                  # or the test shows nothing of them
 
 
+@pytest.mark.parametrize("E,D,Fh,counts", [(5, 72, 40, [128, 0, 129, 1, 60]), (3, 256, 64, [0, 300, 0]),
+                                           (4, 136, 200, [1, 127, 128, 257]), (2, 64, 10, [40, 90]),
+                                           (40, 96, 24, [3] * 39 + [200])])
+def test_tiles_of_the_experts_rows(E, D, Fh, counts):
+    """Shares of no row, one row, a tile's 128 and one more; inner sizes that end inside a piece of K
+    and a tile of columns; every gate and activation; identity pairs behind the experts' are not
+    written."""
+    from gpt_fast_amd.ops import routed_experts as RE
+    g = torch.Generator().manual_seed(D)
+    top, n = 3, (sum(counts) + 7 + 2) // 3
+    pairs = n * top
+    ids = torch.tensor([e for e, c in enumerate(counts) for _ in range(c)] + [E] * (pairs - sum(counts)), dtype=torch.int32)
+    chosen = ids[torch.randperm(pairs, generator=g)].view(n, top).to(DEV)
+    offsets, order, place = RE.expert_order(chosen, E + 1)
+    assert offsets[:E + 1].tolist() == [sum(counts[:e]) for e in range(E + 1)]
+    tiles = RE.expert_tiles(offsets, E, pairs)
+    listed = [t for t in tiles.tolist() if t[0] >= 0]
+    assert listed == [[e, sum(counts[:e]) + i] for e, c in enumerate(counts) for i in range(0, c, 128)]
+    x = torch.randn(n, D, generator=g).bfloat16()
+    w = (torch.randn(E, 2 * Fh, D, generator=g) * 0.3).bfloat16()
+    xs = x.double()[(order.cpu() // top).long()]
+    args = (x.to(DEV), order, top)
+    for act, gated, limit in ((None, False, None), ("silu", False, None), ("gelu", False, None), ("silu", True, None),
+                              ("gelu_tanh", True, None), ("clamped_swish", True, 0.9)):
+        got = RE.expert_tile_product(*args, w.to(DEV), offsets, tiles, pairs, act, gated, limit).double().cpu()
+        for e, c in enumerate(counts):
+            lo = sum(counts[:e])
+            z = xs[lo:lo + c] @ w[e].double().T
+            f = {None: lambda v: v, "silu": P.silu, "gelu": torch.nn.functional.gelu, "gelu_tanh": P.gelu_tanh}
+            if act == "clamped_swish":
+                a, u = z[:, :Fh].clamp(max=limit), z[:, Fh:].clamp(-limit, limit)
+                z = a * torch.sigmoid(1.702 * a) * (u + 1)
+            else:
+                z = f[act](z[:, :Fh]) * z[:, Fh:] if gated else f[act](z)
+            if c:
+                assert rel_err(got[lo:lo + c], z) < 1e-2, (act, gated, e)
+    # rows in their own order (a second product)
+    rows = torch.randn(pairs, D, generator=g).bfloat16()
+    got = RE.expert_tile_product(rows.to(DEV), None, 1, w.to(DEV), offsets, tiles, pairs).double().cpu()
+    for e, c in enumerate(counts):
+        lo = sum(counts[:e])
+        if c:
+            assert rel_err(got[lo:lo + c], rows[lo:lo + c].double() @ w[e].double().T) < 1e-2
+
+
 def test_the_correction_moves_the_choice_and_not_the_weights():
     part, rt, w, mlp = _mixture(4, 2, 2, 64, 32, 1.0, None, "float32")
     part.correction.copy_(torch.tensor([0.0, 0.0, 0.0, 0.0, 5.0, 5.0]))     # both identity experts, always
