@@ -266,7 +266,7 @@ def _stack(width: int, n_layers: int, ff: int, expert_ff: int, shared_ff: int, k
         left_scale=1.0, right_scale=1.0)
     moe = MoeMlp(experts=32, identity=2, top=4, ff=expert_ff, limit=7.0, shared_ff=shared_ff, shared_limit=7.0)
     layers = tuple(PitenexLayer(pair, DenseMlp(ff) if i % 4 == 3 else moe) for i in range(n_layers))
-    return PitenexConfig(vocab=vocab, width=width, norm_eps=1e-6, buckets=65521, mul_prev=31, mul_cur=7,
+    return PitenexConfig(vocab=vocab, width=width, norm_eps=1e-6, buckets=65521, mul_prev=8191, mul_cur=131,
                          residual_mult=0.5, logit_scale=1.0, layers=layers)
 
 

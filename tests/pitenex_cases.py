@@ -52,7 +52,7 @@ CASES = {
     ]),
     # one head on either side, one tap (no convolution), no rotation, ranks that are no multiples of
     # eight and a rank of one, every expert chosen, no identity and no shared expert
-    "B": _model(104, 211, 1e-6, (64, 31, 7), 1.0, 1.0, [
+    "B": _model(104, 211, 1e-6, (64, 29, 13), 1.0, 1.0, [
         _layer(_left(1, 1, 20, 12, 7, None, 0.4), _right(1, 1, 12, 40, 1, (5, 1)), (1.0, 1.0), _dense(60)),
         _layer(_left(8, 8, 8, 24, 33, (4, 50.0), 0.35), _right(8, 1, 20, 10, 5, (1, 13)), (0.5, 1.5),
                _moe(4, 0, 4, 24, 0.5)),
@@ -94,14 +94,14 @@ def random_case(seed):
         if r < 0.4:
             mlp = _dense(rng.choice([96, 128, 200]))
         elif r < 0.9:
-            experts, identity = rng.choice([4, 9, 16]), rng.choice([0, 1, 2, 5])
+            experts, identity = rng.choice([4, 9, 20]), rng.choice([0, 1, 2, 5])
             mlp = _moe(experts, identity, rng.randint(1, 4), rng.choice([32, 40, 64]), rng.choice([0.7, 2.0]),
                        None if rng.random() < 0.2 else (rng.choice([32, 72]), rng.choice([0.5, 1.5])))
         else:
             mlp = None
         layers.append(_layer(left, right, (rng.choice([0.7, 1.0, 1.3]), rng.choice([0.8, 1.0, 1.2])), mlp))
     return _model(width, rng.choice([263, 500, 1000]), rng.choice([1e-5, 1e-6]),
-                  (rng.choice([61, 509, 1024]), rng.choice([3, 31]), rng.choice([1, 7])),
+                  (rng.choice([61, 521, 1024]), rng.choice([3, 29]), rng.choice([1, 5])),
                   rng.choice([0.5, 0.9]), rng.choice([0.5, 1.0]), layers)
 
 
